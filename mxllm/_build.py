@@ -141,6 +141,9 @@ def build(force: bool = False, jobs: int = 8, verbose: bool = False) -> str:
     hip_flags = [
         "-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-munsafe-fp-atomics",
         "-ffp-contract=fast", "-Wno-unused-result", f"-I{CSRC}", f"-I{os.path.join(CSRC, 'kernels')}",
+        # no packed-f32 VALU forms (v_pk_{add,mul,fma}_f32): some have given wrong results on gfx950 now
+        # and then; the host pass does not know the feature and says so (harmless)
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     ]
     cxx_flags = [
         "-O3", "-std=c++17", "-fPIC", "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1", "-DTORCH_API_INCLUDE_EXTENSION_H",
