@@ -2,7 +2,7 @@
 // hipExtStreamCreateWithCUMask runs on, and the HBM bandwidth an AdamW-shaped
 // streaming kernel reaches when confined to that subset.
 //
-// Build: hipcc -O3 --offload-arch=gfx950 bench/cu_mask_probe.hip -o build/cu_mask_probe
+// Build: hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops bench/cu_mask_probe.hip -o build/cu_mask_probe
 // Prints one JSON line per mask.
 #include <hip/hip_runtime.h>
 #include <hip/hip_ext.h>
