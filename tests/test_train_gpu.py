@@ -60,7 +60,12 @@ def test_overlapped_adamw_bitwise(gpu, gdt, sched, monkeypatch):
             monkeypatch.setenv("MXLLM_ADAMW_LAG", "1")
         if ovl and sched == "cus":
             monkeypatch.setenv("MXLLM_ADAMW_CUS", "mod8:2")
-        tr = _ddp_trainer(gpu, cfg, 11, overlap_optimizer=ovl, grad_dtype=gdt)
+        try:
+            tr = _ddp_trainer(gpu, cfg, 11, overlap_optimizer=ovl, grad_dtype=gdt)
+        except RuntimeError as e:
+            if sched == "cus" and "hipExtStreamCreateWithCUMask" in str(e):
+                pytest.skip(f"this machine grants no CU-masked stream: {e}")
+            raise
         assert tr.overlap_optimizer == ovl
         if ovl and sched == "lag":
             assert tr._lag == 1
