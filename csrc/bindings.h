@@ -4,6 +4,10 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 
+namespace mx {
+struct ConvRope;
+}
+
 extern "C" {
 // rmsnorm.hip
 int mx_rmsnorm_fwd(const uint16_t* x, const uint16_t* res, const uint16_t* w, uint16_t* y,
@@ -138,4 +142,28 @@ int64_t mx_swiglu_lora_ws(int T, int F, int nrb);
 int mx_swiglu_lora(int bwd, const uint16_t* gu, const uint16_t* dm, uint16_t* out, int64_t ldo, const uint16_t* V,
                    int64_t ldv, int nrb, int pad, float alpha, float* ws, int T, int F, hipStream_t stream);
 int mx_lora_xtg(const int64_t* desc, int np, int T, float alpha, int accumulate, float* ws, hipStream_t stream);
+// hybrid.hip / mingru.hip / chunk_attn.hip / attn_fwd.hip SEG: f32 != 0 = float activations, else bf16
+int mx_embed_rows(const int64_t* ids, const void* w, int f32, float* out, int64_t T, int W, int V, hipStream_t stream);
+int mx_group_norm(const void* delta, int64_t ldd, float* h, const float* w, void* y, int64_t ldy, int f32, int64_t T,
+                  int W, int groups, float eps, hipStream_t stream);
+int mx_conv_rope_prefill(const mx::ConvRope* a, int f32, const int32_t* rowpos, const int32_t* rowseq,
+                         const int32_t* seqs, int T, hipStream_t stream);
+int mx_conv_rope_decode(const mx::ConvRope* a, int f32, const int32_t* pos, const int32_t* slots, int B,
+                        hipStream_t stream);
+int mx_poly_norm(const void* z, int64_t ldz, const float* coef, void* y, int f32, int64_t T, int F, float eps,
+                 hipStream_t stream);
+int mx_attn_combine(const float* ml, const float* po, const uint16_t* gate, int64_t ldg, uint16_t* out, int B, int H,
+                    int D, int E, int nsplit, hipStream_t stream);
+int mx_attn_fwd_seg(const uint16_t* q, const uint16_t* k, const uint16_t* v, const int32_t* blocks, int nblk,
+                    const uint16_t* gate, int64_t ldg, uint16_t* o, int T, int Hq, int Hkv, int D, int E, float scale,
+                    hipStream_t stream);
+int mx_chunk_attn(const void* q, int64_t qh, int64_t qt, const void* k, const void* v, int64_t kh, int64_t vh, int Dp,
+                  int Ep, const int32_t* pos, const int32_t* slots, const int32_t* bt, int maxb, int block,
+                  const void* gate, int64_t ldg, void* out, int f32, int64_t rows, int H, int G, int D, int E,
+                  int chunk, float scale, hipStream_t stream);
+int mx_mingru_scan(const void* x, int64_t ldx, int f32, const float* bias, const int32_t* chunks, int nc,
+                   const int32_t* seqs, int nseq, int multi, float* prod, float* part, float* state, void* y, int W,
+                   hipStream_t stream);
+int mx_mingru_step(const void* x, int64_t ldx, int f32, const float* bias, const int32_t* slots, float* state, void* y,
+                   int B, int W, hipStream_t stream);
 }

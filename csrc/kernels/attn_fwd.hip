@@ -73,11 +73,23 @@ __device__ __forceinline__ u16x4 tr_read(const char* p) {
 // tile's V landed) and E (after PV: every wave is done with the V slot the next tile restages).
 // Tile kt issues K(kt + 2) and V(kt + 1) during its QK^T steps, so a K tile has two tiles of MFMAs
 // to land and a V tile one and a half, where the symmetric 2-slot ring gives both one.
-template <int D, bool CAUSAL, int NW, bool PROF = false, int R = 2, bool SR = false>
+// SEG (ragged prompts): q / k / v are [heads, T, D] over the rows of all sequences and every
+// workgroup takes its query block from a table of segments that attend only to themselves (a chunk
+// of one sequence).  The softmax has a sink (a key of score 0 without a value: the running max starts
+// at 0 and the sum at 1), and the output (E <= D dims per head) is multiplied by sigmoid(gate).
+struct AttnSeg {
+  const int4* blocks;    // [gridDim / Hq] (first row of the segment, its rows, query block, -)
+  const uint16_t* gate;  // [T, ldg]: head h's gate at column h * E
+  int64_t ldg;
+  int T, E;
+};
+
+template <int D, bool CAUSAL, int NW, bool PROF = false, int R = 2, bool SR = false, bool SEG = false>
 __global__ void __launch_bounds__(64 * NW, 8 / NW)
 attn_fwd_kernel(const uint16_t* __restrict__ Q, const uint16_t* __restrict__ K, const uint16_t* __restrict__ V,
                 uint16_t* __restrict__ O, float* __restrict__ LSE, int B, int Hq, int Hkv, int S, int Sk,
-                int causal_off, float sl, int ldo, int flags, uint32_t* __restrict__ prof = nullptr) {
+                int causal_off, float sl, int ldo, int flags, uint32_t* __restrict__ prof = nullptr,
+                AttnSeg seg = {}) {
   // PROF (diagnostic build, MXLLM_ATTN_PROF=1): per-wave s_memtime cycle sums of the tile phases
   uint32_t ph[6] = {0, 0, 0, 0, 0, 0};
   uint64_t tp0 = 0, t_entry = 0, t_loop = 0;
@@ -106,13 +118,20 @@ attn_fwd_kernel(const uint16_t* __restrict__ Q, const uint16_t* __restrict__ K, 
   const int nqb = (S + BM - 1) / BM;
   const int BH = B * Hq;
   const int bid = xcd_balance(blockIdx.x, gridDim.x, BH, Hq / Hkv);
-  const int qb = nqb - 1 - bid / BH;
+  int qb = nqb - 1 - bid / BH;
   const int bh = bid % BH;
   const int b = bh / Hq, h = bh % Hq;
   const int hk = h / (Hq / Hkv);
-  const uint16_t* Qp = Q + ((size_t)(b * Hq + h) * S) * D;
-  const uint16_t* Kp = K + ((size_t)(b * Hkv + hk) * Sk) * D;
-  const uint16_t* Vp = V + ((size_t)(b * Hkv + hk) * Sk) * D;
+  size_t row0 = 0;
+  size_t qo = (size_t)(b * Hq + h) * S, ko = (size_t)(b * Hkv + hk) * Sk;
+  if constexpr (SEG) {
+    const int4 sg = seg.blocks[bid / BH];
+    row0 = sg.x, S = sg.y, Sk = sg.y, qb = sg.z;
+    qo = (size_t)h * seg.T + row0, ko = (size_t)hk * seg.T + row0;
+  }
+  const uint16_t* Qp = Q + qo * D;
+  const uint16_t* Kp = K + ko * D;
+  const uint16_t* Vp = V + ko * D;
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);  // provably wave-uniform (no divergent branches)
   // 8 waves = two per SIMD from the same workgroup: give the upper four priority 1 so the pair
@@ -189,7 +208,7 @@ attn_fwd_kernel(const uint16_t* __restrict__ Q, const uint16_t* __restrict__ K, 
     for (int j = 0; j < 16; ++j) o[d][j] = 0.f;
   // m_i: the (deferred) running max of this row in the log2 domain of the scaled
   // scores; l_i: running sum of exp2(s*sl - m_i)
-  float m_i = -1e30f, l_i = 0.f;
+  float m_i = SEG ? 0.f : -1e30f, l_i = SEG && hh == 0 ? 1.f : 0.f;
 
   // Loop-invariant LDS byte addresses.  The XOR swizzle of a row depends only on
   // row & 15, so for every (n, s2) k-step and both ring buffers a fragment address
@@ -434,7 +453,35 @@ attn_fwd_kernel(const uint16_t* __restrict__ Q, const uint16_t* __restrict__ K, 
     l_tot = __uint_as_float(sw[0]) + __uint_as_float(sw[1]);
   }
   const float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
-  if (qrow < S) {
+  if constexpr (SEG) {
+    if (qrow < S) {
+      const uint16_t* gp = seg.gate + (row0 + qrow) * (size_t)seg.ldg + (size_t)h * seg.E;
+      uint16_t* op = O + (row0 + qrow) * (size_t)ldo + (size_t)h * seg.E;
+      // 4-element accesses when every head's columns start on 8 bytes
+      const bool v4 = ((seg.E | (int)(seg.ldg & 3) | ldo) & 3) == 0 && ((size_t)seg.gate & 7) == 0;
+#pragma unroll
+      for (int db = 0; db < DB; ++db)
+#pragma unroll
+        for (int gq = 0; gq < 4; ++gq) {
+          const int d = db * 32 + 8 * gq + 4 * hh;
+          if (d >= seg.E) continue;
+          u16x4 g4 = {0, 0, 0, 0}, v4o;
+          if (v4) g4 = *reinterpret_cast<const u16x4*>(gp + d);
+          else
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              if (d + j < seg.E) g4[j] = gp[d + j];
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            v4o[j] = f2bf(o[db][4 * gq + j] * inv * __builtin_amdgcn_rcpf(1.f + __expf(-bf2f(g4[j]))));
+          if (v4) *reinterpret_cast<u16x4*>(op + d) = v4o;
+          else
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              if (d + j < seg.E) op[d + j] = v4o[j];
+        }
+    }
+  } else if (qrow < S) {
     uint16_t* op = O + ((size_t)b * S + qrow) * (size_t)ldo + (size_t)h * D;
 #pragma unroll
     for (int db = 0; db < DB; ++db)
@@ -1222,5 +1269,25 @@ extern "C" int mx_attn_fwd(const uint16_t* q, const uint16_t* k, const uint16_t*
   else if (D == 32) { if (causal) FWD(32, true); else FWD(32, false); }
   else return -1;
 #undef FWD
+  return (int)hipGetLastError();
+}
+
+// Ragged prompts (attn_fwd_kernel SEG): q [Hq, T, D], k / v [Hkv, T, D] (unused dims zero), blocks
+// [nblk] query blocks of 128 rows, gate [T, ldg], o [T, Hq * E].
+extern "C" int mx_attn_fwd_seg(const uint16_t* q, const uint16_t* k, const uint16_t* v, const int32_t* blocks,
+                               int nblk, const uint16_t* gate, int64_t ldg, uint16_t* o, int T, int Hq, int Hkv, int D,
+                               int E, float scale, hipStream_t stream) {
+  if (T <= 0 || nblk <= 0) return 0;
+  if (Hkv <= 0 || Hq % Hkv || E <= 0 || E > D || ldg < (int64_t)Hq * E) return -1;
+  const AttnSeg sg{reinterpret_cast<const int4*>(blocks), gate, ldg, T, E};
+  const float sl = scale * 1.4426950408889634f;
+#define FWDS(DD)                                                                                                \
+  attn_fwd_kernel<DD, true, 4, false, 2, false, true><<<nblk * Hq, 256, 0, stream>>>(                           \
+      q, k, v, o, nullptr, 1, Hq, Hkv, T, T, 0, sl, Hq * E, 1, nullptr, sg)
+  if (D == 128) FWDS(128);
+  else if (D == 64) FWDS(64);
+  else if (D == 32) FWDS(32);
+  else return -1;
+#undef FWDS
   return (int)hipGetLastError();
 }

@@ -625,7 +625,8 @@ extern "C" int mx_decode_attn(const uint16_t* q, const uint16_t* kc, const uint1
   if (bt && max_seq % kSplit) return -1;  // a split must lie inside one block
   dim3 grid(nsplit, Hkv, B);
   const float sl = scale * 1.4426950408889634f;
-  if (D == 128) {  // out == nullptr: partials only (the o-projection merges them: skinny_gemm.hip MERGE)
+  // out == nullptr: partials only, merged by the caller (skinny_gemm.hip MERGE, hybrid.hip attn_combine)
+  if (D == 128) {
     // cnt (zeroed [B * Hkv] counters, owned by the caller): the splits merge in-launch
     // MXLLM_DECODE_HANDOFF: hand-off protocol of the in-launch merge (see the kernel; read per call)
     const char* pe = getenv("MXLLM_DECODE_HANDOFF");
@@ -637,11 +638,10 @@ extern "C" int mx_decode_attn(const uint16_t* q, const uint16_t* kc, const uint1
     if (out && !fused) decode_combine_kernel<128><<<B * Hq, 128, 0, stream>>>(part_ml, part_o, out, nsplit);
     return (int)hipGetLastError();
   }
-  if (!out) return -1;
 #define DA(DD)                                                                                                  \
   decode_attn_kernel<DD><<<grid, 256, 0, stream>>>(q, kc, vc, lens, len_off, slots, part_ml, part_o, Hq, Hkv, \
                                                    max_seq, nsplit, sl, bt, maxb);                              \
-  decode_combine_kernel<DD><<<B * Hq, DD, 0, stream>>>(part_ml, part_o, out, nsplit)
+  if (out) decode_combine_kernel<DD><<<B * Hq, DD, 0, stream>>>(part_ml, part_o, out, nsplit)
   if (D == 64) { DA(64); } else if (D == 32) { DA(32); } else return -1;
 #undef DA
   return (int)hipGetLastError();

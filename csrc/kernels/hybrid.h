@@ -1,0 +1,87 @@
+// Shared pieces of the recurrent / chunked-attention model kernels (hybrid.hip, mingru.hip,
+// chunk_attn.hip): element access for bf16 and f32 storage, and the f32 scalar functions.
+// Storage type T is uint16_t (bf16 bits) or float; all arithmetic is f32.
+#pragma once
+
+#include "common.h"
+
+namespace mx {
+
+template <typename T>
+__device__ __forceinline__ float ld1(const T* p) {
+  if constexpr (sizeof(T) == 2) return bf2f(*p);
+  else return *p;
+}
+template <typename T>
+__device__ __forceinline__ void st1(T* p, float v) {
+  if constexpr (sizeof(T) == 2) *p = f2bf(v);
+  else *p = v;
+}
+// VEC consecutive elements (VEC 1, 2, 4 or 8; the address is VEC-element aligned)
+template <int VEC, typename T>
+__device__ __forceinline__ void ldv(const T* p, float (&v)[VEC]) {
+  if constexpr (VEC == 1) {
+    v[0] = ld1(p);
+  } else if constexpr (sizeof(T) == 2) {
+    typedef uint16_t vt __attribute__((ext_vector_type(VEC)));
+    const vt x = *reinterpret_cast<const vt*>(p);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = bf2f(x[i]);
+  } else if constexpr (VEC == 2) {
+    const float2 x = *reinterpret_cast<const float2*>(p);
+    v[0] = x.x;
+    v[1] = x.y;
+  } else {
+#pragma unroll
+    for (int c = 0; c < VEC; c += 4) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(p + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[c + i] = x[i];
+    }
+  }
+}
+template <int VEC, typename T>
+__device__ __forceinline__ void stv(T* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 1) {
+    st1(p, v[0]);
+  } else if constexpr (sizeof(T) == 2) {
+    typedef uint16_t vt __attribute__((ext_vector_type(VEC)));
+    vt x;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) x[i] = f2bf(v[i]);
+    *reinterpret_cast<vt*>(p) = x;
+  } else if constexpr (VEC == 2) {
+    *reinterpret_cast<float2*>(p) = make_float2(v[0], v[1]);
+  } else {
+#pragma unroll
+    for (int c = 0; c < VEC; c += 4) {
+      f32x4 x;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i] = v[c + i];
+      *reinterpret_cast<f32x4*>(p + c) = x;
+    }
+  }
+}
+
+// the f32-storage kernels take the library exponential, the bf16 ones the hardware exp2 form
+template <typename T>
+__device__ __forceinline__ float exp_t(float x) {
+  if constexpr (sizeof(T) == 2) return __expf(x);
+  else return expf(x);
+}
+template <typename T>
+__device__ __forceinline__ float sigmoid_t(float x) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+  else return 1.f / (1.f + expf(-x));
+}
+
+// one minGRU token: s <- (1 - z) s + z c, z = sigmoid(zp), c = up + 1/2 (up >= 0) or sigmoid(up)
+template <typename T>
+__device__ __forceinline__ void mingru_gate(float zp, float up, float& keep, float& add) {
+  const float z = sigmoid_t<T>(zp);
+  const float c = up >= 0.f ? up + 0.5f : sigmoid_t<T>(up);
+  keep = 1.f - z;
+  add = z * c;
+}
+
+}  // namespace mx

@@ -1,0 +1,423 @@
+// Row kernels of the recurrent / chunked-attention decoders for gfx950:
+//   * embed_rows   : token rows of the embedding table into the f32 residual stream;
+//   * group_norm   : (residual add +) RMS norm in equal consecutive groups, f32 residual;
+//   * conv_rope    : short causal convolution over time on the q / k / v projections, rotation
+//                    of interleaved pairs, and the KV-cache / convolution-tail stores (prompt
+//                    rows of several sequences at once, or one token per sequence);
+//   * poly_norm    : the polynomial-of-norms activation;
+//   * attn_combine : split-K decode partials merged with the softmax sink and the output gate.
+// Storage type T: bf16 (uint16_t) or float; every reduction, angle and product is f32.
+#include <algorithm>
+
+#include "conv_rope.h"
+#include "hybrid.h"
+
+namespace mx {
+
+// ------------------------------------------------------------------ embedding -> f32 rows
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) embed_rows_kernel(const int64_t* __restrict__ ids, const T* __restrict__ w,
+                                                         float* __restrict__ out, int64_t n, int W, int V) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  const int nv = W / VEC;
+  const int64_t row = i / nv;
+  const int c = (int)(i % nv) * VEC;
+  int64_t id = ids[row];
+  id = id < 0 ? 0 : (id >= V ? V - 1 : id);  // ids are checked on the host; stays in the table either way
+  float v[VEC];
+  ldv<VEC>(w + id * W + c, v);
+  stv<VEC>(out + row * W + c, v);
+}
+
+// ------------------------------------------------------------------ grouped RMS norm
+// The norm of a row in G equal parts is an RMS norm of G rows: one unit = one (row, part), held in
+// registers by TPU threads (a wave or a workgroup).  h (f32, row stride W) += delta when given.
+template <typename T, int TPU, int VEC>
+__global__ void __launch_bounds__(TPU < 256 ? 256 : TPU)
+    group_norm_kernel(const T* __restrict__ delta, int64_t ldd, float* __restrict__ h, const float* __restrict__ w,
+                      T* __restrict__ y, int64_t ldy, int64_t units, int groups, int gs, float eps) {
+  constexpr int ITERS = 16 / VEC;
+  __shared__ float scratch[16];
+  const int64_t unit = TPU < 256 ? (int64_t)blockIdx.x * (256 / TPU) + threadIdx.x / TPU : (int64_t)blockIdx.x;
+  const bool on = unit < units;
+  const int t = threadIdx.x % TPU;
+  const int64_t row = on ? unit / groups : 0;
+  const int g0 = on ? (int)(unit % groups) * gs : 0;
+  float* hp = h + row * (int64_t)groups * gs + g0;
+  const T* dp = delta ? delta + row * ldd + g0 : nullptr;
+  float v[ITERS][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int c = (it * TPU + t) * VEC;
+    if (on && c < gs) {
+      ldv<VEC>(hp + c, v[it]);
+      if (dp) {
+        float d[VEC];
+        ldv<VEC>(dp + c, d);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[it][j] += d[j];
+        stv<VEC>(hp + c, v[it]);
+      }
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss += v[it][j] * v[it][j];
+    }
+  }
+  ss = TPU == 64 ? wave_sum(ss) : block_sum(ss, scratch);
+  const float rs = 1.f / sqrtf(ss / (float)gs + eps);
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int c = (it * TPU + t) * VEC;
+    if (on && c < gs) {
+      float g[VEC], o[VEC];
+      ldv<VEC>(w + g0 + c, g);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = v[it][j] * rs * g[j];
+      stv<VEC>(y + row * ldy + g0 + c, o);
+    }
+  }
+}
+
+// ------------------------------------------------------------------ convolution + rotation
+
+// section and channel of flat vector index f: sec 0 q, 1 k, 2 v; head; d0; ch = flat channel
+template <int VEC>
+__device__ __forceinline__ void conv_where(const ConvRope& a, int f, int& sec, int& head, int& d0, int& ch, int& dim) {
+  const int nd = (a.D + VEC - 1) / VEC, ne = (a.E + VEC - 1) / VEC;
+  if (f < a.H * nd) {
+    sec = 0, head = f / nd, d0 = (f % nd) * VEC, dim = a.D;
+    ch = head * a.D + d0;
+  } else if (f < (a.H + a.G) * nd) {
+    f -= a.H * nd;
+    sec = 1, head = f / nd, d0 = (f % nd) * VEC, dim = a.D;
+    ch = a.H * a.D + head * a.D + d0;
+  } else {
+    f -= (a.H + a.G) * nd;
+    sec = 2, head = f / ne, d0 = (f % ne) * VEC, dim = a.E;
+    ch = (a.H + a.G) * a.D + head * a.E + d0;
+  }
+}
+
+// values of channels [ch, ch + n) of a row; channels past n are 0 (n = VEC except at an odd head end)
+template <int VEC, typename T>
+__device__ __forceinline__ void ldn(const T* p, int n, float (&v)[VEC]) {
+  if constexpr (VEC >= 4) {
+    ldv<VEC>(p, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = i < n ? ld1(p + i) : 0.f;
+  }
+}
+template <int VEC, typename T>
+__device__ __forceinline__ void stn(T* p, int n, const float (&v)[VEC]) {
+  if constexpr (VEC >= 4) {
+    stv<VEC>(p, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i)
+      if (i < n) st1(p + i, v[i]);
+  }
+}
+
+// rotate and store the convolved channels y of (row, position p, cache slot); keep: into the cache
+template <int VEC, typename T>
+__device__ __forceinline__ void conv_finish(const ConvRope& a, int sec, int head, int d0, int n, int64_t row, int p,
+                                            int slot, bool keep, float (&y)[VEC]) {
+  if (sec < 2) {
+#pragma unroll
+    for (int i = 0; i + 1 < VEC; i += 2) {
+      const int d = d0 + i;
+      if (d + 1 < a.rd) {
+        const float c = a.cosb[(int64_t)p * (a.rd >> 1) + (d >> 1)], s = a.sinb[(int64_t)p * (a.rd >> 1) + (d >> 1)];
+        const float u = y[i], v = y[i + 1];
+        y[i] = u * c - v * s;
+        y[i + 1] = v * c + u * s;
+      }
+    }
+  }
+  const int Wp = sec < 2 ? a.Dp : a.Ep;
+  T* out = reinterpret_cast<T*>(sec == 0 ? a.q : sec == 1 ? a.k : a.v);
+  if (out) {
+    out += sec == 0 ? head * a.qh + row * a.qt : sec == 1 ? head * a.kh + row * a.kt : head * a.vh + row * a.vt;
+    stn<VEC>(out + d0, n, y);
+    const int dim = sec < 2 ? a.D : a.E;
+    if (d0 + VEC >= dim)  // the head's last channels: its padding too
+      for (int d = dim; d < Wp; ++d) st1(out + d, 0.f);
+  }
+  if (sec == 0) return;
+  T* cache = reinterpret_cast<T*>(sec == 1 ? a.kc : a.vc);
+  if (cache && keep)
+    stn<VEC>(cache + kv_row(a.bt, a.maxb, a.block, slot, a.G, head, p % a.chunk) * Wp + d0, n, y);
+}
+
+// prompt rows: rowpos [T] position, rowseq [T] sequence, seqs [n, 2] = (slot or -1, length).
+// One thread walks RUN consecutive rows of VEC channels with the last taps - 1 rows in registers.
+constexpr int kConvRun = 8;
+template <int VEC, typename T, int TAPS>
+__global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, const int32_t* __restrict__ rowpos,
+                                                                const int32_t* __restrict__ rowseq,
+                                                                const int32_t* __restrict__ seqs, int T_, int nvec) {
+  const int f = blockIdx.x * 256 + threadIdx.x;
+  if (f >= nvec) return;
+  int sec, head, d0, ch, dim;
+  conv_where<VEC>(a, f, sec, head, d0, ch, dim);
+  const int n = min(VEC, dim - d0);
+  const T* x = reinterpret_cast<const T*>(a.x) + ch;
+  const int C = (a.H + a.G) * a.D + a.G * a.E;
+  const int taps = TAPS ? TAPS : a.taps;
+  const int r0 = blockIdx.y * kConvRun, r1 = min(T_, r0 + kConvRun);
+  if constexpr (TAPS > 0) {
+    float wt[TAPS][VEC], win[TAPS][VEC];  // win[j]: row r - (TAPS - 1) + j
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) wt[j][i] = i < n ? a.w[(int64_t)(ch + i) * TAPS + j] : 0.f;
+#pragma unroll
+    for (int j = 1; j < TAPS; ++j) {
+      const int r = r0 - TAPS + j;
+      if (r >= 0) ldn<VEC>(x + r * a.ldx, n, win[j]);
+      else
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) win[j][i] = 0.f;
+    }
+    for (int r = r0; r < r1; ++r) {
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) win[j][i] = win[j + 1][i];
+      ldn<VEC>(x + r * a.ldx, n, win[TAPS - 1]);
+      const int p = rowpos[r], sq = rowseq[r], slot = seqs[2 * sq], S = seqs[2 * sq + 1];
+      float y[VEC];
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) y[i] = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+        if (p >= TAPS - 1 - j)  // the row TAPS - 1 - j back is of this sequence
+#pragma unroll
+          for (int i = 0; i < VEC; ++i) y[i] += wt[j][i] * win[j][i];
+      if (slot >= 0 && a.ring && p >= S - taps)
+        stn<VEC>(reinterpret_cast<T*>(a.ring) + ((int64_t)slot * taps + p % taps) * C + ch, n, win[TAPS - 1]);
+      conv_finish<VEC, T>(a, sec, head, d0, n, r, p, slot, slot >= 0 && p >= S / a.chunk * a.chunk, y);
+    }
+  } else {
+    for (int r = r0; r < r1; ++r) {
+      const int p = rowpos[r], sq = rowseq[r], slot = seqs[2 * sq], S = seqs[2 * sq + 1];
+      float y[VEC], u[VEC];
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) y[i] = 0.f;
+      for (int j = 0; j < taps; ++j) {
+        const int back = taps - 1 - j;
+        if (p < back) continue;
+        ldn<VEC>(x + (int64_t)(r - back) * a.ldx, n, u);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) y[i] += (i < n ? a.w[(int64_t)(ch + i) * taps + j] : 0.f) * u[i];
+      }
+      if (slot >= 0 && a.ring && p >= S - taps) {
+        ldn<VEC>(x + (int64_t)r * a.ldx, n, u);
+        stn<VEC>(reinterpret_cast<T*>(a.ring) + ((int64_t)slot * taps + p % taps) * C + ch, n, u);
+      }
+      conv_finish<VEC, T>(a, sec, head, d0, n, r, p, slot, slot >= 0 && p >= S / a.chunk * a.chunk, y);
+    }
+  }
+}
+
+// one token per sequence: earlier projected values come from the ring
+template <int VEC, typename T>
+__global__ void __launch_bounds__(64) conv_rope_decode_kernel(ConvRope a, const int32_t* __restrict__ pos,
+                                                              const int32_t* __restrict__ slots, int nvec) {
+  const int f = blockIdx.x * 64 + threadIdx.x;
+  if (f >= nvec) return;
+  int sec, head, d0, ch, dim;
+  conv_where<VEC>(a, f, sec, head, d0, ch, dim);
+  const int n = min(VEC, dim - d0), b = blockIdx.y, p = pos[b], slot = slots[b];
+  const int C = (a.H + a.G) * a.D + a.G * a.E;
+  T* ring = reinterpret_cast<T*>(a.ring) + (int64_t)slot * a.taps * C + ch;
+  float u[VEC], y[VEC];
+  ldn<VEC>(reinterpret_cast<const T*>(a.x) + (int64_t)b * a.ldx + ch, n, u);
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) y[i] = (i < n ? a.w[(int64_t)(ch + i) * a.taps + a.taps - 1] : 0.f) * u[i];
+  for (int back = 1; back < a.taps && back <= p; ++back) {
+    float o[VEC];
+    ldn<VEC>(ring + (int64_t)((p - back) % a.taps) * C, n, o);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) y[i] += (i < n ? a.w[(int64_t)(ch + i) * a.taps + a.taps - 1 - back] : 0.f) * o[i];
+  }
+  stn<VEC>(ring + (int64_t)(p % a.taps) * C, n, u);
+  conv_finish<VEC, T>(a, sec, head, d0, n, b, p, slot, true, y);
+}
+
+// ------------------------------------------------------------------ PolyNorm
+// y = a N(z) + b N(z^2) + c N(z^3) + e, N over the whole row; coef = (a, b, c, e)
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) poly_norm_kernel(const T* __restrict__ z, int64_t ldz,
+                                                        const float* __restrict__ coef, T* __restrict__ y, int F,
+                                                        float eps) {
+  __shared__ float scratch[16];
+  const T* zp = z + (int64_t)blockIdx.x * ldz;
+  T* yp = y + (int64_t)blockIdx.x * F;
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  for (int c = threadIdx.x * VEC; c < F; c += 256 * VEC) {
+    float v[VEC];
+    ldv<VEC>(zp + c, v);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const float q = v[i] * v[i];
+      s1 += q;
+      s2 += q * q;
+      s3 += q * q * q;
+    }
+  }
+  s1 = block_sum(s1, scratch);
+  s2 = block_sum(s2, scratch);
+  s3 = block_sum(s3, scratch);
+  const float inv = 1.f / (float)F;
+  const float k1 = coef[0] / sqrtf(s1 * inv + eps), k2 = coef[1] / sqrtf(s2 * inv + eps),
+              k3 = coef[2] / sqrtf(s3 * inv + eps), e = coef[3];
+  for (int c = threadIdx.x * VEC; c < F; c += 256 * VEC) {
+    float v[VEC], o[VEC];
+    ldv<VEC>(zp + c, v);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) o[i] = ((k3 * v[i] + k2) * v[i] + k1) * v[i] + e;
+    stv<VEC>(yp + c, o);
+  }
+}
+
+// ------------------------------------------------------------------ decode combine: sink + gate
+// out[b, h E + d] = sigmoid(gate[b, h E + d]) * sum_s 2^(m_s - M) o_s[d] / (2^-M + sum_s 2^(m_s - M) l_s)
+// with M = max(0, m_s): the added 1 of the denominator is a key of score 0 without a value.
+__global__ void __launch_bounds__(128) attn_combine_kernel(const float* __restrict__ ml, const float* __restrict__ po,
+                                                           const uint16_t* __restrict__ gate, int64_t ldg,
+                                                           uint16_t* __restrict__ out, int H, int D, int E,
+                                                           int nsplit) {
+  const int64_t bh = blockIdx.x, b = bh / H;
+  const int h = (int)(bh % H), d = threadIdx.x;
+  if (d >= E) return;
+  const float* m = ml + bh * nsplit * 2;
+  const float gv = bf2f(gate[b * ldg + (int64_t)h * E + d]);
+  float M = 0.f;
+  for (int s = 0; s < nsplit; ++s) M = fmaxf(M, m[2 * s]);
+  float L = __builtin_amdgcn_exp2f(-M), acc = 0.f;
+  for (int s = 0; s < nsplit; ++s) {
+    const float ms = m[2 * s];
+    if (ms == -INFINITY) continue;
+    const float wg = __builtin_amdgcn_exp2f(ms - M);
+    L += wg * m[2 * s + 1];
+    acc += wg * po[(bh * nsplit + s) * D + d];
+  }
+  out[b * (int64_t)H * E + (int64_t)h * E + d] = f2bf(acc / L * sigmoid_t<uint16_t>(gv));
+}
+
+}  // namespace mx
+
+using namespace mx;
+
+extern "C" int mx_embed_rows(const int64_t* ids, const void* w, int f32, float* out, int64_t T, int W, int V,
+                             hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (W <= 0 || V <= 0) return -1;
+  const int vec = W % 4 == 0 ? 4 : 1;
+  const int64_t n = T * (W / vec);
+  const unsigned grid = (unsigned)((n + 255) / 256);
+#define EM(TT, VV) embed_rows_kernel<TT, VV><<<grid, 256, 0, stream>>>(ids, (const TT*)w, out, n, W, V)
+  if (f32) { if (vec == 4) EM(float, 4); else EM(float, 1); }
+  else { if (vec == 4) EM(uint16_t, 4); else EM(uint16_t, 1); }
+#undef EM
+  return (int)hipGetLastError();
+}
+
+extern "C" int mx_group_norm(const void* delta, int64_t ldd, float* h, const float* w, void* y, int64_t ldy, int f32,
+                             int64_t T, int W, int groups, float eps, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (groups <= 0 || W % groups) return -1;
+  const int gs = W / groups;
+  if (gs > 16384) return -1;
+  const int64_t units = T * groups;
+  const bool v4 = gs % 4 == 0 && (!delta || ldd % 4 == 0) && ldy % 4 == 0;
+#define GN(TT, TPU, VV)                                                                                      \
+  group_norm_kernel<TT, TPU, VV>                                                                             \
+      <<<(unsigned)(TPU == 64 ? (units + 3) / 4 : units), TPU == 64 ? 256 : TPU, 0, stream>>>(               \
+          (const TT*)delta, ldd, h, w, (TT*)y, ldy, units, groups, gs, eps)
+#define GNT(TT)                                                                                              \
+  if (v4) { if (gs <= 512) GN(TT, 64, 4); else if (gs <= 4096) GN(TT, 256, 4); else GN(TT, 1024, 4); }       \
+  else { if (gs <= 1024) GN(TT, 64, 1); else if (gs <= 4096) GN(TT, 256, 1); else GN(TT, 1024, 1); }
+  if (f32) { GNT(float) } else { GNT(uint16_t) }
+#undef GNT
+#undef GN
+  return (int)hipGetLastError();
+}
+
+static int conv_check(const ConvRope& a) {
+  if (a.taps < 1 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.D <= 0 || a.E <= 0 || a.rd < 0 || a.rd > a.D || a.rd % 2 ||
+      a.chunk <= 0 || a.Dp < a.D || a.Ep < a.E || (a.kc && (!a.vc || !a.bt || a.block <= 0)))
+    return -1;
+  return 0;
+}
+template <int VEC>
+static int conv_nvec(const ConvRope& a) {
+  return (a.H + a.G) * ((a.D + VEC - 1) / VEC) + a.G * ((a.E + VEC - 1) / VEC);
+}
+static bool conv_v8(const ConvRope& a) {
+  return a.D % 8 == 0 && a.E % 8 == 0 && a.ldx % 8 == 0 && a.Dp % 8 == 0 && a.Ep % 8 == 0 && a.qh % 8 == 0 &&
+         a.qt % 8 == 0 && a.kh % 8 == 0 && a.kt % 8 == 0 && a.vh % 8 == 0 && a.vt % 8 == 0;
+}
+
+
+extern "C" int mx_conv_rope_prefill(const ConvRope* pa, int f32, const int32_t* rowpos, const int32_t* rowseq,
+                                    const int32_t* seqs, int T, hipStream_t stream) {
+  if (T <= 0) return 0;
+  const ConvRope& a = *pa;
+  if (conv_check(a)) return -1;
+#define CP(VV, TT, TP)                                                                             \
+  conv_rope_prefill_kernel<VV, TT, TP><<<dim3((conv_nvec<VV>(a) + 255) / 256, (T + kConvRun - 1) / kConvRun), 256, \
+                                         0, stream>>>(a, rowpos, rowseq, seqs, T, conv_nvec<VV>(a))
+#define CPT(VV, TT)                                                                                \
+  if (a.taps == 4) CP(VV, TT, 4); else if (a.taps == 3) CP(VV, TT, 3); else if (a.taps == 2) CP(VV, TT, 2); \
+  else CP(VV, TT, 0)
+  if (f32) { CPT(2, float); }
+  else if (conv_v8(a)) { CPT(8, uint16_t); }
+  else { CPT(2, uint16_t); }
+#undef CPT
+#undef CP
+  return (int)hipGetLastError();
+}
+
+extern "C" int mx_conv_rope_decode(const ConvRope* pa, int f32, const int32_t* pos, const int32_t* slots, int B,
+                                   hipStream_t stream) {
+  if (B <= 0) return 0;
+  const ConvRope& a = *pa;
+  if (conv_check(a) || !a.ring) return -1;
+#define CD(VV, TT)                                                                                          \
+  conv_rope_decode_kernel<VV, TT><<<dim3((conv_nvec<VV>(a) + 63) / 64, B), 64, 0, stream>>>(a, pos, slots, \
+                                                                                            conv_nvec<VV>(a))
+  if (f32) CD(2, float);
+  else if (conv_v8(a)) CD(8, uint16_t);
+  else CD(2, uint16_t);
+#undef CD
+  return (int)hipGetLastError();
+}
+
+extern "C" int mx_poly_norm(const void* z, int64_t ldz, const float* coef, void* y, int f32, int64_t T, int F,
+                            float eps, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (F <= 0) return -1;
+  const unsigned g = (unsigned)T;
+  if (f32) {
+    if (F % 4 == 0 && ldz % 4 == 0)
+      poly_norm_kernel<float, 4><<<g, 256, 0, stream>>>((const float*)z, ldz, coef, (float*)y, F, eps);
+    else poly_norm_kernel<float, 1><<<g, 256, 0, stream>>>((const float*)z, ldz, coef, (float*)y, F, eps);
+  } else {
+    if (F % 8 == 0 && ldz % 8 == 0)
+      poly_norm_kernel<uint16_t, 8><<<g, 256, 0, stream>>>((const uint16_t*)z, ldz, coef, (uint16_t*)y, F, eps);
+    else poly_norm_kernel<uint16_t, 1><<<g, 256, 0, stream>>>((const uint16_t*)z, ldz, coef, (uint16_t*)y, F, eps);
+  }
+  return (int)hipGetLastError();
+}
+
+extern "C" int mx_attn_combine(const float* ml, const float* po, const uint16_t* gate, int64_t ldg, uint16_t* out,
+                               int B, int H, int D, int E, int nsplit, hipStream_t stream) {
+  if (B <= 0) return 0;
+  if (E > 128 || E > D || nsplit < 1) return -1;
+  attn_combine_kernel<<<B * H, 128, 0, stream>>>(ml, po, gate, ldg, out, H, D, E, nsplit);
+  return (int)hipGetLastError();
+}
