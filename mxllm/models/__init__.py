@@ -1,26 +1,53 @@
 from .config import LlamaConfig, PRESETS, get_config  # noqa: F401
 from .llama import Llama, FusedLinear  # noqa: F401
 from .hf import is_hf_dir, load_hf_config, load_hf_llama, save_hf_llama  # noqa: F401
+from .revesun import Revesun, RevesunConfig, load_revesun, save_revesun  # noqa: F401
+from . import revesun as _revesun
+
+# config.json "architecture" -> (config reader, weight loader); directories without the key are
+# Hugging Face Llama checkpoints (mxllm/models/hf.py)
+ARCHITECTURES = {"Revesun": (_revesun.load_config, load_revesun)}
+# config class -> model class of a preset
+MODEL_CLASSES = {LlamaConfig: Llama, RevesunConfig: Revesun}
 
 
-def model_config(name: str) -> LlamaConfig:
-    """A preset name (``llama3.1-8b`` ...) or a Hugging Face Llama directory."""
-    return load_hf_config(name) if is_hf_dir(name) else get_config(name)
+def architecture(path: str) -> str | None:
+    """The ``architecture`` a model directory names (None: a Hugging Face Llama directory)."""
+    import json
+    import os
+
+    with open(os.path.join(path, "config.json")) as f:
+        a = json.load(f).get("architecture")
+    if a is not None and a not in ARCHITECTURES:
+        raise ValueError(f"{path}: unknown architecture {a!r}; have {sorted(ARCHITECTURES)}")
+    return a
+
+
+def model_config(name: str):
+    """A preset name (``llama3.1-8b`` ...) or a model directory (config.json + safetensors)."""
+    if not is_hf_dir(name):
+        return get_config(name)
+    a = architecture(name)
+    return ARCHITECTURES[a][0](name) if a else load_hf_config(name)
 
 
 def build_model(name: str, *, device=None, dtype=None, lora_r: int = 0, lora_alpha: float = 16.0, seed: int = 0,
-                **kw) -> Llama:
-    """Random-init preset, or the weights of a Hugging Face Llama directory."""
+                **kw):
+    """Random-init preset, or the weights of a model directory (Hugging Face Llama, or one of
+    ``ARCHITECTURES`` by its config.json)."""
     import torch
 
     dtype = dtype or torch.bfloat16
+    kw.update(device=device, dtype=dtype, lora_r=lora_r, lora_alpha=lora_alpha, seed=seed)
     if is_hf_dir(name):
-        return load_hf_llama(name, device=device, dtype=dtype, lora_r=lora_r, lora_alpha=lora_alpha, seed=seed, **kw)
-    return Llama(get_config(name), device=device, dtype=dtype, lora_r=lora_r, lora_alpha=lora_alpha, seed=seed, **kw)
+        a = architecture(name)
+        return (ARCHITECTURES[a][1] if a else load_hf_llama)(name, **kw)
+    cfg = get_config(name)
+    return MODEL_CLASSES[type(cfg)](cfg, **kw)
 
 
 def tokenizer_path_for(name: str, explicit: str | None = None) -> str | None:
-    """An explicit tokenizer.json, else the one shipped in a Hugging Face model directory."""
+    """An explicit tokenizer.json, else the one shipped in a model directory."""
     import os
 
     if explicit:

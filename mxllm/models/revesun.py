@@ -1,0 +1,328 @@
+"""Revesun: a decoder whose layers are minGRU recurrences or chunked attention, with a grouped
+RMS norm, an f32 residual stream and PolyNorm feed-forwards (MI355X serving layout).
+
+Every size and constant comes from ``config.json`` (``RevesunConfig.from_json``); layers differ
+freely in kind and sizes.  The projections that read a layer's normed input are one GEMM each:
+z | u | gate of a minGRU, q | k | v | gate of an attention layer.  ``rows`` runs the layer stack
+over a row layout of mxllm/ops/hybrid.py: whole prompts of several sequences, or one token each.
+
+Weights: the projections in the model dtype (bf16, or f32 for a true-f32 run); norm weights,
+biases, convolution taps and activation coefficients in f32.  The embedding is also the head.
+"""
+from __future__ import annotations
+
+import dataclasses
+import json
+import math
+import os
+from dataclasses import dataclass
+
+import torch
+import torch.nn as nn
+
+from ..ops import hybrid as hops
+from ..ops import linear
+from ..ops.hybrid import AttnShape, PromptRows
+from .config import PRESETS
+from .llama import FusedLinear
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    """One layer.  ``mingru``: ``width`` channels.  ``attention``: ``attn`` shape, ``rot_base``.
+    ``ff``: feed-forward width, 0 for a layer without one."""
+
+    kind: str
+    width: int = 0
+    attn: AttnShape | None = None
+    rot_base: float = 10000.0
+    ff: int = 0
+
+    def n_params(self, h: int) -> int:
+        n = h
+        if self.kind == "mingru":
+            n += 4 * h * self.width + 2 * self.width
+        else:
+            a = self.attn
+            n += h * (a.conv_channels + 2 * a.heads * a.vdim) + a.conv_channels * a.taps
+        return n + (h + 2 * h * self.ff + 4 if self.ff else 0)
+
+
+@dataclass(frozen=True)
+class RevesunConfig:
+    name: str
+    vocab_size: int
+    hidden: int
+    layers: tuple
+    norm_groups: int = 1
+    norm_eps: float = 1e-5
+    max_seq_len: int = 131072  # the design has no limit of its own: the longest the rotation tables go
+    bos_id: int = 256
+    eos_id: int = -1           # no end token: generation ends by length or a request's stop ids
+
+    @property
+    def n_layers(self) -> int:
+        return len(self.layers)
+
+    def n_params(self) -> int:
+        return sum(s.n_params(self.hidden) for s in self.layers) + self.vocab_size * self.hidden + self.hidden
+
+    def replace(self, **kw) -> "RevesunConfig":
+        return dataclasses.replace(self, **kw)
+
+    @staticmethod
+    def from_json(d: dict, name: str = "revesun") -> "RevesunConfig":
+        specs = []
+        for i, e in enumerate(d["layers"]):
+            mx, mlp = e["mixer"], e.get("mlp")
+            if mlp is not None and mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not supported")
+            ff = int(mlp["ff"]) if mlp is not None else 0
+            if e["type"] == "mingru":
+                specs.append(LayerSpec("mingru", width=int(mx["width"]), ff=ff))
+            elif e["type"] == "attention":
+                a = AttnShape(heads=int(mx["heads"]), kv_heads=int(mx["kv_heads"]), dim=int(mx["dim"]),
+                              vdim=int(mx["vdim"]), taps=int(mx["conv"]), chunk=int(mx["mask"]["size"]),
+                              rot_dims=int(mx["rot"]["dims"]), scale=float(mx["scale"]))
+                if a.heads % a.kv_heads or a.rot_dims % 2 or a.rot_dims > a.dim or a.chunk < 1 or a.taps < 1:
+                    raise ValueError(f"layer {i}: inconsistent attention sizes {a}")
+                specs.append(LayerSpec("attention", attn=a, rot_base=float(mx["rot"]["base"]), ff=ff))
+            else:
+                raise ValueError(f"layer {i}: unknown layer type {e['type']!r}")
+        if d["width"] % d["norm"]["groups"]:
+            raise ValueError(f"width {d['width']} does not split into {d['norm']['groups']} norm groups")
+        return RevesunConfig(name=name, vocab_size=int(d["vocab"]), hidden=int(d["width"]), layers=tuple(specs),
+                             norm_groups=int(d["norm"]["groups"]), norm_eps=float(d["norm"]["eps"]),
+                             bos_id=256 if d["vocab"] > 256 else 0)
+
+    def to_json(self) -> dict:
+        layers = []
+        for s in self.layers:
+            if s.kind == "mingru":
+                mx = {"width": s.width}
+            else:
+                a = s.attn
+                mx = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "conv": a.taps,
+                      "mask": {"size": a.chunk}, "rot": {"base": s.rot_base, "dims": a.rot_dims}, "scale": a.scale}
+            layers.append({"type": s.kind, "mixer": mx, "mlp": {"kind": "dense", "ff": s.ff} if s.ff else None})
+        return {"architecture": "Revesun", "vocab": self.vocab_size, "width": self.hidden, "layers": layers,
+                "norm": {"eps": self.norm_eps, "groups": self.norm_groups}}
+
+
+class RevesunLayer(nn.Module):
+    """``wx``: the projections of the normed input (z | u | gate, or q | k | v | gate); ``wo``: the
+    mixer's output; ``wup`` / ``wdown``: the feed-forward."""
+
+    def __init__(self, spec: LayerSpec, h: int, *, dtype, device):
+        super().__init__()
+        self.spec = spec
+        kw = dict(dtype=dtype, device=device)
+
+        def f32(*shape, value=0.0):
+            return nn.Parameter(torch.full(shape, value, dtype=torch.float32, device=device))
+
+        self.norm1 = f32(h, value=1.0)
+        if spec.kind == "mingru":
+            self.wx = FusedLinear(h, [spec.width] * 3, **kw)
+            self.bias = f32(2 * spec.width)
+            self.wo = FusedLinear(spec.width, [h], **kw)
+        else:
+            a = spec.attn
+            self.wx = FusedLinear(h, [a.heads * a.dim, a.kv_heads * a.dim, a.kv_heads * a.vdim, a.heads * a.vdim], **kw)
+            self.conv = f32(a.conv_channels, a.taps)
+            self.wo = FusedLinear(a.heads * a.vdim, [h], **kw)
+        if spec.ff:
+            self.norm2 = f32(h, value=1.0)
+            self.wup = FusedLinear(h, [spec.ff], **kw)
+            self.act = f32(4)
+            self.wdown = FusedLinear(spec.ff, [h], **kw)
+
+
+class Revesun(nn.Module):
+    def __init__(self, cfg: RevesunConfig, *, device=None, dtype=torch.bfloat16, seed: int = 0, init: bool = True,
+                 lora_r: int = 0, lora_alpha: float = 16.0):
+        super().__init__()
+        if lora_r:
+            raise NotImplementedError("Revesun has no LoRA adapters (serving only)")
+        device = torch.device(device) if device is not None else torch.device("cpu")
+        self.cfg = cfg
+        self.dtype = dtype
+        self.tok_emb = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden, dtype=dtype, device=device))
+        self.layers = nn.ModuleList([RevesunLayer(s, cfg.hidden, dtype=dtype, device=device) for s in cfg.layers])
+        self.final_norm = nn.Parameter(torch.ones(cfg.hidden, dtype=torch.float32, device=device))
+        # index of each layer among the layers that keep keys / a recurrent state
+        count = {"attention": 0, "mingru": 0}
+        self.kind_index = []
+        for s in cfg.layers:
+            self.kind_index.append(count[s.kind])
+            count[s.kind] += 1
+        self._rope: dict = {}
+        if init:
+            self.reset_parameters(seed)
+        self.requires_grad_(False)
+
+    @torch.no_grad()
+    def reset_parameters(self, seed: int = 0):
+        """Random weights that keep the residual stream near unit scale."""
+        gen = torch.Generator(device=self.tok_emb.device)
+        gen.manual_seed(seed)
+        self.tok_emb.normal_(0.0, 1.0 / math.sqrt(self.cfg.hidden), generator=gen)
+        for layer in self.layers:
+            for m in layer.children():
+                m.weight.normal_(0.0, 1.0 / math.sqrt(m.in_features), generator=gen)
+            if layer.spec.kind == "mingru":
+                layer.bias.normal_(0.0, 0.5, generator=gen)
+            else:
+                layer.conv.normal_(0.0, 0.2, generator=gen)
+                layer.conv[:, -1] += 1.0
+            if layer.spec.ff:
+                layer.act.copy_(torch.tensor([0.5, 0.3, 0.2, 0.1]))
+
+    @property
+    def head_weight(self) -> torch.Tensor:
+        return self.tok_emb
+
+    # ------------------------------------------------------------------ rotation tables
+    def rope(self, spec: LayerSpec, n: int) -> tuple[torch.Tensor, torch.Tensor]:
+        """Tables of at least ``n`` positions for an attention layer (shared by layers alike)."""
+        key = (spec.attn.rot_dims, spec.rot_base)
+        have = self._rope.get(key)
+        if have is None or have[0].shape[0] < n:
+            n = max(n, 256)
+            have = hops.pair_rope_tables(n, *key, device=self.tok_emb.device)
+            self._rope[key] = have
+        return have
+
+    def prepare(self, max_seq: int) -> None:
+        """Size the rotation tables once (their storage must not move under a captured graph)."""
+        for s in self.cfg.layers:
+            if s.kind == "attention":
+                self.rope(s, max_seq)
+
+    # ------------------------------------------------------------------ the layer stack
+    def _norm_proj(self, delta, h, gamma, lin) -> torch.Tensor:
+        return lin(hops.group_norm(delta, h, gamma, self.cfg.norm_groups, self.cfg.norm_eps, self.dtype))
+
+    def rows(self, ids: torch.Tensor, rows, tap=None) -> torch.Tensor:
+        """Final normed hidden rows of token ``ids`` [T] laid out as ``rows``.  ``tap(i, h)``: the
+        residual stream after layer i (diagnostics)."""
+        n = rows.max_len if rows.decode else max(rows.lens)
+        h = hops.embed_rows(ids, self.tok_emb)
+        delta = None
+        for i, layer in enumerate(self.layers):
+            s, j = layer.spec, self.kind_index[i]
+            x = self._norm_proj(delta, h, layer.norm1, layer.wx)
+            if s.kind == "mingru":
+                y = hops.min_gru(x, layer.bias, rows, j)
+            else:
+                cos, sin = self.rope(s, n)
+                y = hops.sink_attention(x, layer.conv, cos, sin, s.attn, rows, j)
+            delta = layer.wo(y)
+            if s.ff:
+                z = self._norm_proj(delta, h, layer.norm2, layer.wup)
+                delta = layer.wdown(hops.poly_norm(z, layer.act, self.cfg.norm_eps))
+            if tap is not None:
+                tap(i, h + delta.float())
+        return hops.group_norm(delta, h, self.final_norm, self.cfg.norm_groups, self.cfg.norm_eps, self.dtype)
+
+    @torch.no_grad()
+    def hidden_states(self, ids: torch.Tensor, tap=None) -> torch.Tensor:
+        """ids [B, S] -> final normed hidden [B * S, H]; nothing is cached."""
+        B, S = ids.shape
+        return self.rows(ids.reshape(-1), PromptRows([S] * B, self.tok_emb.device), tap)
+
+    @torch.no_grad()
+    def forward(self, ids: torch.Tensor) -> torch.Tensor:
+        """Logits [B, S, V] of whole sequences."""
+        return linear(self.hidden_states(ids), self.head_weight).view(*ids.shape, -1)
+
+    def num_params(self, trainable_only: bool = False) -> int:
+        return 0 if trainable_only else sum(p.numel() for p in self.parameters())
+
+
+# ------------------------------------------------------------------ checkpoints
+def load_config(path: str) -> RevesunConfig:
+    with open(os.path.join(path, "config.json")) as f:
+        return RevesunConfig.from_json(json.load(f), name=os.path.basename(os.path.normpath(path)))
+
+
+def name_map(cfg: RevesunConfig) -> dict[str, list[str]]:
+    """mxllm parameter -> the checkpoint tensors whose rows it concatenates."""
+    m = {"tok_emb": ["embed"], "final_norm": ["final.norm"]}
+    for i, s in enumerate(cfg.layers):
+        p, q = f"layers.{i}.", f"l{i}."
+        m[p + "norm1"] = [q + "norm1"]
+        m[p + "wo.weight"] = [q + "mix.o"]
+        if s.kind == "mingru":
+            m[p + "wx.weight"] = [q + "mix." + x for x in ("z", "x", "g")]
+            m[p + "bias"] = [q + "mix.z.b", q + "mix.x.b"]
+        else:
+            m[p + "wx.weight"] = [q + "mix." + x for x in ("q", "k", "v", "g")]
+            m[p + "conv"] = [q + f"mix.{x}.conv" for x in ("q", "k", "v")]
+        if s.ff:
+            m.update({p + "norm2": [q + "norm2"], p + "wup.weight": [q + "mlp.up"], p + "act": [q + "mlp.act"],
+                      p + "wdown.weight": [q + "mlp.down"]})
+    return m
+
+
+@torch.no_grad()
+def load_revesun(path: str, *, device=None, dtype: torch.dtype = torch.bfloat16, **kw) -> Revesun:
+    """The model of a directory with ``config.json`` and safetensors (strict: every tensor present,
+    fitting, and used)."""
+    from .hf import HFReader
+
+    cfg = load_config(path)
+    kw.pop("seed", None)
+    model = Revesun(cfg, device=device, dtype=dtype, init=False, **kw)
+    rd = HFReader(path)
+    params = dict(model.named_parameters())
+    for name, srcs in name_map(cfg).items():
+        rd.fill_(params[name].data, srcs)
+    rd.check_all_used(False)
+    return model
+
+
+@torch.no_grad()
+def save_revesun(model: Revesun, path: str) -> str:
+    """Write ``config.json`` + ``model.safetensors`` readable by :func:`load_revesun` (bf16 tensors)."""
+    from safetensors.torch import save_file
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(model.cfg.to_json(), f, indent=1)
+    params, out = dict(model.named_parameters()), {}
+    for name, srcs in name_map(model.cfg).items():
+        t = params[name].detach().to("cpu", torch.bfloat16)
+        for src, part in zip(srcs, t.split(_rows_of(model, name, srcs))):
+            out[src] = part.contiguous()
+    fn = os.path.join(path, "model.safetensors")
+    save_file(out, fn)
+    return fn
+
+
+def _rows_of(model: Revesun, name: str, srcs: list[str]) -> list[int]:
+    """Row counts of the checkpoint tensors stacked in parameter ``name``."""
+    params = dict(model.named_parameters())
+    if len(srcs) == 1:
+        return [params[name].shape[0]]
+    layer = model.layers[int(name.split(".")[1])]
+    if name.endswith("bias"):
+        return [layer.spec.width] * 2
+    return layer.wx.splits[:len(srcs)]
+
+
+# ------------------------------------------------------------------ presets
+def _stack(n: int, width: int, heads: int, kv: int, dim: int, chunk: int, ff: int, base: float) -> tuple:
+    """n layers, a minGRU and an attention layer in turn, each with a feed-forward."""
+    attn = AttnShape(heads, kv, dim, dim, 4, chunk, dim // 2, 1.0 / math.sqrt(dim))
+    return tuple(LayerSpec("attention", attn=attn, rot_base=base, ff=ff) if i % 2 else
+                 LayerSpec("mingru", width=width, ff=ff) for i in range(n))
+
+
+PRESETS["revesun-tiny"] = RevesunConfig("revesun-tiny", 320, 64, _stack(4, 96, 4, 2, 16, 24, 160, 1e4), norm_groups=2)
+# projection and feed-forward sizes of the Llama presets of the same name (two feed-forward matrices of
+# 1.5x the width in place of three)
+PRESETS["revesun-1b"] = RevesunConfig("revesun-1b", 128256, 2048, _stack(16, 2048, 16, 4, 128, 4096, 12288, 5e5),
+                                      norm_groups=8)
+PRESETS["revesun-8b"] = RevesunConfig("revesun-8b", 128256, 4096, _stack(32, 4096, 32, 8, 128, 4096, 21504, 5e5),
+                                      norm_groups=8)

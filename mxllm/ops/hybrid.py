@@ -1,0 +1,310 @@
+"""Ops of decoders that mix recurrent and chunked-attention layers: grouped RMS norm on an f32
+residual, the minGRU recurrence, convolved + pair-rotated attention with a softmax sink and an
+output gate, PolyNorm; and the row layouts they run on.
+
+``PromptRows``: the concatenated tokens of several sequences from their first token on.
+``TokenRows``: one token for each of several sequences (a decode step, graph-capturable).
+Both carry where a layer's cached rows and state live (``SeqCaches``), so a model's layer loop is
+the same for both.
+
+GPU: csrc/kernels/hybrid.hip, mingru.hip, chunk_attn.hip, attn_fwd.hip (SEG) and decode.hip.
+CPU tensors: plain PyTorch (the CPU test suite).
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+
+import numpy as np
+import torch
+
+from ._ext import native, use_native
+
+MFMA_MAX_DIM = 128  # widest head of the MFMA attention kernels
+MFMA_MAX_REP = 16   # query heads per key head in the split-K decode kernels
+
+
+@dataclass(frozen=True)
+class AttnShape:
+    """One attention layer's constants.  ``chunk``: position i sees only keys of its own run of
+    ``chunk`` positions; ``rot_dims`` of ``dim`` are rotated (interleaved pairs)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+    chunk: int
+    rot_dims: int
+    scale: float
+
+    @property
+    def conv_channels(self) -> int:
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+    def mfma(self, dtype: torch.dtype) -> bool:
+        """bf16 heads the matrix-core attention kernels take; the rest runs on chunk_attn.hip."""
+        return (dtype == torch.bfloat16 and max(self.dim, self.vdim) <= MFMA_MAX_DIM
+                and self.heads // self.kv_heads <= MFMA_MAX_REP)
+
+    def row_dims(self, dtype: torch.dtype) -> tuple[int, int]:
+        """Stored width of a key and of a value row: the MFMA kernels take one width of 32, 64 or
+        128 for both (unused dims zero), the others whole 16-byte pieces."""
+        if self.mfma(dtype):
+            w = next(x for x in (32, 64, 128) if x >= max(self.dim, self.vdim))
+            return w, w
+        a = 16 // dtype.itemsize
+        return (self.dim + a - 1) // a * a, (self.vdim + a - 1) // a * a
+
+
+@dataclass
+class SeqCaches:
+    """What sequences keep between steps.  ``k`` / ``v``: per attention layer, paged pools
+    [blocks, kv_heads, block, width]; a layer keeps position p at row p % chunk, so a slot's
+    blocks cover at most one chunk.  ``conv``: per attention layer [slots, taps, channels], the
+    projected values of position p at p % taps.  ``rec``: per recurrent layer f32 [slots, width]."""
+
+    k: list
+    v: list
+    bt: torch.Tensor
+    conv: list
+    rec: list
+
+
+def pair_rope_tables(n: int, dims: int, base: float, device=None) -> tuple[torch.Tensor, torch.Tensor]:
+    """cos / sin f32 [n, dims / 2] of position * base^(-2i / dims) (angles in f64, rounded once)."""
+    i = torch.arange(dims // 2, dtype=torch.float64, device=device)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64, device=device), -2.0 * i / max(dims, 1))
+    a = torch.arange(n, dtype=torch.float64, device=device)[:, None] * f[None]
+    return a.cos().float().contiguous(), a.sin().float().contiguous()
+
+
+# ------------------------------------------------------------------ row layouts
+class PromptRows:
+    """Rows of several prompts, each from position 0; ``slots`` None: nothing is kept."""
+
+    decode = False
+
+    def __init__(self, lens: list[int], device, slots: list[int] | None = None, caches: SeqCaches | None = None):
+        self.lens, self.device, self.caches = list(lens), device, caches if slots is not None else None
+        self.slots = list(slots) if slots is not None else [-1] * len(lens)
+        self.offs = np.concatenate([[0], np.cumsum(self.lens)]).astype(np.int64)
+        self.T = int(self.offs[-1])
+        self._tables: dict = {}
+        pos = np.concatenate([np.arange(n, dtype=np.int32) for n in self.lens])
+        seq = np.repeat(np.arange(len(self.lens), dtype=np.int32), self.lens)
+        self.rowpos, self.rowseq = self._up(pos), self._up(seq)
+        self.seqs = self._up(np.array([self.slots, self.lens], dtype=np.int32).T)
+
+    def _up(self, a: np.ndarray) -> torch.Tensor:
+        return torch.from_numpy(np.ascontiguousarray(a)).to(self.device)
+
+    def attn_blocks(self, chunk: int) -> torch.Tensor:
+        """int32 [n, 4] query blocks of 128 rows of every (sequence, chunk) segment, longest first."""
+        key = ("attn", chunk)
+        if key not in self._tables:
+            rows = []
+            for o, n in zip(self.offs, self.lens):
+                for s in range(0, n, chunk):
+                    m = min(chunk, n - s)
+                    rows += [(int(o) + s, m, qb, 0) for qb in range((m + 127) // 128)]
+            rows.sort(key=lambda r: -r[2])
+            self._tables[key] = self._up(np.array(rows, dtype=np.int32))
+        return self._tables[key]
+
+    def scan_tables(self, width: int):
+        """(chunks int32 [n, 4] = first row, rows, sequence, last-of-sequence; seqs int32 [m, 3] =
+        slot, first chunk, chunks; whether any sequence has several) for a scan of ``width`` channels:
+        chunks short enough to fill the GPU with waves."""
+        L = max(16, min(128, self.T * width // (256 * 2048)))
+        L = 1 << (L.bit_length() - 1)
+        key = ("scan", L)
+        if key not in self._tables:
+            ch, sq = [], []
+            for i, (o, n) in enumerate(zip(self.offs, self.lens)):
+                c0 = len(ch)
+                for s in range(0, n, L):
+                    ch.append((int(o) + s, min(L, n - s), i, int(s + L >= n)))
+                sq.append((self.slots[i], c0, len(ch) - c0))
+            self._tables[key] = (self._up(np.array(ch, dtype=np.int32)), self._up(np.array(sq, dtype=np.int32)),
+                                 any(s[2] > 1 for s in sq))
+        return self._tables[key]
+
+
+class TokenRows:
+    """One token per sequence: ``pos`` / ``slots`` int32 [B] on the device, ``max_len`` a host bound
+    on pos + 1."""
+
+    decode = True
+
+    def __init__(self, pos: torch.Tensor, slots: torch.Tensor, max_len: int, caches: SeqCaches):
+        self.pos, self.slots, self.max_len, self.caches = pos, slots, max_len, caches
+        self._local: dict = {}
+
+    def chunk_pos(self, chunk: int) -> torch.Tensor:
+        """Position inside the chunk = index of the newest cached row."""
+        if chunk >= self.max_len:
+            return self.pos
+        if chunk not in self._local:
+            self._local[chunk] = torch.remainder(self.pos, chunk)
+        return self._local[chunk]
+
+
+# ------------------------------------------------------------------ ops
+def embed_rows(ids: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """Token rows of the embedding table as the f32 residual stream."""
+    if use_native(w):
+        return native().embed_rows(ids.contiguous(), w)
+    return w[ids].float()
+
+
+def group_norm(delta: torch.Tensor | None, h: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
+               dtype: torch.dtype) -> torch.Tensor:
+    """h (f32, in place) += delta; returns the RMS norm of h in ``groups`` equal parts, times w."""
+    if use_native(h):
+        return native().group_norm(delta, h, w, groups, eps, dtype == torch.float32)
+    if delta is not None:
+        h += delta.float()
+    p = h.view(h.shape[0], groups, -1)
+    return ((p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).view_as(h) * w).to(dtype)
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
+    """a N(z) + b N(z^2) + c N(z^3) + e with N the RMS norm over the row; coef = (a, b, c, e)."""
+    if use_native(z):
+        return native().poly_norm(z, coef, eps)
+    x = z.float()
+    y = coef[3]
+    for i in range(3):
+        p = x ** (i + 1)
+        y = y + coef[i] * p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)
+    return y.to(z.dtype)
+
+
+def min_gru(x: torch.Tensor, bias: torch.Tensor, rows, layer: int) -> torch.Tensor:
+    """Gated recurrence over the rows of ``rows``: x [T, 3W] = z | u | g projections, bias f32 [2W]
+    (z | u); recurrent layer ``layer``'s state is read and written in ``rows.caches``."""
+    W = x.shape[1] // 3
+    state = rows.caches.rec[layer] if rows.caches is not None else None
+    if use_native(x):
+        if rows.decode:
+            return native().mingru_step(x, bias, rows.slots, state)
+        chunks, seqs, multi = rows.scan_tables(W)
+        return native().mingru_scan(x, bias, chunks, seqs, multi, state)
+    z, u, g = x.float().split(W, 1)
+    z = torch.sigmoid(z + bias[:W])
+    u = u + bias[W:]
+    add, keep = z * torch.where(u >= 0, u + 0.5, torch.sigmoid(u)), 1 - z
+    s = torch.empty_like(z)
+    if rows.decode:
+        idx = rows.slots.long()
+        s = keep * state[idx] + add
+        state[idx] = s
+    else:
+        for i, n in enumerate(rows.lens):
+            cur = torch.zeros(W)
+            for t in range(int(rows.offs[i]), int(rows.offs[i]) + n):
+                cur = keep[t] * cur + add[t]
+                s[t] = cur
+            if state is not None:
+                state[rows.slots[i]] = cur
+    return (s * torch.nn.functional.silu(g)).to(x.dtype)
+
+
+def sink_attention(x: torch.Tensor, conv: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor, sh: AttnShape, rows,
+                   layer: int) -> torch.Tensor:
+    """x [T, q | k | v | gate] projections -> gated attention output [T, heads * vdim]: causal
+    convolution of q, k, v over time, rotation of q and k, attention inside chunks with one added to
+    the softmax's denominator, times sigmoid(gate).  ``conv`` f32 [channels, taps]."""
+    C = sh.conv_channels
+    gate = x[:, C:]
+    H, G, D, E = sh.heads, sh.kv_heads, sh.dim, sh.vdim
+    c = rows.caches
+    if not use_native(x):
+        return _sink_attention_ref(x, conv, cos, sin, sh, rows, layer)
+    ops = native()
+    Dp, Ep = sh.row_dims(x.dtype)
+    args = (x, conv, cos, sin, sh.rot_dims, H, G, D, E)
+    if not rows.decode:
+        keep = (c.k[layer], c.v[layer], c.bt, c.conv[layer]) if c is not None else ()
+        q, k, v = ops.conv_rope_prefill(*args, Dp, Ep, rows.rowpos, rows.rowseq, rows.seqs, sh.chunk, *keep)
+        if sh.mfma(x.dtype):
+            return ops.attn_seg(q, k, v, rows.attn_blocks(sh.chunk), gate, E, sh.scale)
+        return ops.chunk_attn(q, k, v, rows.rowpos, gate, D, E, sh.chunk, sh.scale)
+    q = ops.conv_rope_decode(*args, rows.pos, rows.slots, sh.chunk, c.k[layer], c.v[layer], c.bt, c.conv[layer])
+    return decode_sink_attention(q, gate, sh, rows, layer)
+
+
+def decode_sink_attention(q: torch.Tensor, gate: torch.Tensor, sh: AttnShape, rows: TokenRows,
+                          layer: int) -> torch.Tensor:
+    """One query per sequence over the cached rows of its chunk (the new token's already stored)."""
+    ops, c = native(), rows.caches
+    if sh.mfma(q.dtype):
+        ml, po = ops.decode_attn_partials(q, c.k[layer], c.v[layer], rows.chunk_pos(sh.chunk), rows.slots,
+                                          min(rows.max_len, sh.chunk), sh.scale, 1, c.bt)
+        return ops.attn_combine(ml, po, gate, sh.vdim)
+    return ops.chunk_attn(q, c.k[layer], c.v[layer], rows.pos, gate, sh.dim, sh.vdim, sh.chunk, sh.scale, rows.slots,
+                          c.bt)
+
+
+# ------------------------------------------------------------------ CPU attention
+def _sink_attention_ref(x, conv, cos, sin, sh: AttnShape, rows, layer: int) -> torch.Tensor:
+    H, G, D, E, C, n = sh.heads, sh.kv_heads, sh.dim, sh.vdim, sh.conv_channels, sh.taps
+    c = rows.caches
+    bt = c.bt.tolist() if c is not None else None
+
+    def place(slot, p):  # cache block and row of position p
+        r = p % sh.chunk
+        blk = c.k[layer].shape[2]
+        return bt[slot][r // blk], r % blk
+
+    def rot(t, p):  # [heads, D] at position p
+        t = t.clone()
+        k = sh.rot_dims
+        a, b = t[:, 0:k:2].clone(), t[:, 1:k:2].clone()
+        t[:, 0:k:2], t[:, 1:k:2] = a * cos[p] - b * sin[p], b * cos[p] + a * sin[p]
+        return t
+
+    def attend(q, ks, vs):  # q [H, D], ks [L, G, D], vs [L, G, E]
+        ks, vs = ks.repeat_interleave(H // G, 1), vs.repeat_interleave(H // G, 1)
+        s = torch.matmul(ks.transpose(0, 1), q[:, :, None])[..., 0] * sh.scale  # [H, L]
+        m = s.amax(1, keepdim=True).clamp_min(0)
+        e = torch.exp(s - m)
+        w = e / (e.sum(1, keepdim=True) + torch.exp(-m))
+        return torch.matmul(w[:, None], vs.transpose(0, 1))[:, 0].reshape(-1)
+
+    def token(u, hist, p):  # newest value u [C], hist: earlier ones newest first
+        y = conv[:, n - 1] * u
+        for back, o in enumerate(hist[:n - 1], 1):
+            y = y + conv[:, n - 1 - back] * o
+        return (rot(y[:H * D].view(H, D), p).to(x.dtype).float(), rot(y[H * D:(H + G) * D].view(G, D), p),
+                y[(H + G) * D:].view(G, E))
+
+    out = torch.empty(x.shape[0], H * E)
+    u = x[:, :C].float()
+    if rows.decode:
+        for b, (p, s) in enumerate(zip(rows.pos.tolist(), rows.slots.tolist())):
+            hist = [c.conv[layer][s, (p - j) % n].float() for j in range(1, n) if p >= j]
+            q, k, v = token(u[b], hist, p)
+            c.conv[layer][s, p % n] = x[b, :C]
+            blk, r = place(s, p)
+            c.k[layer][blk, :, r, :D], c.v[layer][blk, :, r, :E] = k.to(x.dtype), v.to(x.dtype)
+            at = [place(s, j) for j in range(p // sh.chunk * sh.chunk, p + 1)]
+            out[b] = attend(q, torch.stack([c.k[layer][i, :, j, :D] for i, j in at]).float(),
+                            torch.stack([c.v[layer][i, :, j, :E] for i, j in at]).float())
+    else:
+        for i, L in enumerate(rows.lens):
+            o, s = int(rows.offs[i]), rows.slots[i]
+            ks, vs = [], []
+            for p in range(L):
+                q, k, v = token(u[o + p], [u[o + p - j] for j in range(1, n) if p >= j], p)
+                ks.append(k.to(x.dtype).float())
+                vs.append(v.to(x.dtype).float())
+                lo = p // sh.chunk * sh.chunk
+                out[o + p] = attend(q, torch.stack(ks[lo:]), torch.stack(vs[lo:]))
+                if c is not None:
+                    if p >= L - n:
+                        c.conv[layer][s, p % n] = x[o + p, :C]
+                    if p >= L // sh.chunk * sh.chunk:
+                        blk, r = place(s, p)
+                        c.k[layer][blk, :, r, :D], c.v[layer][blk, :, r, :E] = k.to(x.dtype), v.to(x.dtype)
+    return (out * torch.sigmoid(x[:, C:].float())).to(x.dtype)

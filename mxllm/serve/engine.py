@@ -5,6 +5,9 @@ This replaces the reference's remote API offload: ``get_model_response``
 over HTTP, one blocking request per prompt.  Here every rank
 serves its own shard of prompts from its own GPU, batched.
 
+What depends on the model class (caches, prompt pass, decode step) is its steps object
+(mxllm/serve/steps.py); this file is slots, scheduling, graphs and sampling.
+
 MI355X-first sizing: the KV cache (mxllm/serve/kvcache.py) is a pool of
 256-token blocks per layer addressed through a per-slot block table.  Static
 mode gives every slot max_seq positions (70B: 320 KiB/token, 16 slots x 8k
@@ -40,23 +43,8 @@ from dataclasses import dataclass, field
 import torch
 
 from .. import ops
-from ..models.llama import FusedLinear
 from ..ops import decode as dops
 
-_SWIGLU_FUSED = os.environ.get("MXLLM_SWIGLU_FUSED", "1") != "0"  # A/B switch (bench/serve_bench.py)
-_NORM_FUSED = os.environ.get("MXLLM_NORM_FUSED", "1") != "0"  # A/B switch: RMSNorm in the decode GEMM prologue
-_ROPE_FUSED = os.environ.get("MXLLM_ROPE_FUSED", "1") != "0"  # A/B switch: RoPE + cache append in the QKV epilogue
-# the split-K attention merge in the o-projection GEMM's prologue (decode rows <= 4): OFF by
-# default -- measured 8B decode, same box: batch 1 3.424 vs 3.433 ms (a wash), batch 4 4.113 vs
-# 3.841 ms (the prologue slows the weight stream more than the combine launch costs;
-# archive/profiles/r3d_decode_merge_ab.md).  MXLLM_MERGE_FUSED=1 turns it on.
-_MERGE_FUSED = os.environ.get("MXLLM_MERGE_FUSED", "0") == "1"
-# Small-batch decode: while the (latency-bound) attention runs, a side-stream kernel reads
-# the layer's o-projection weight so the o-projection GEMM streams it from the Infinity
-# Cache instead of HBM (MXLLM_DECODE_PREFETCH=1; up to PREFETCH_MAX_B rows).  Measured
-# slower (fork/join + competing reads; archive/profiles/r3g/README.md): off by default.
-_PREFETCH = os.environ.get("MXLLM_DECODE_PREFETCH", "0") == "1"
-PREFETCH_MAX_B = 8
 log = logging.getLogger("mxllm.engine")
 
 
@@ -114,6 +102,7 @@ class Engine:
                 self.tp = None
         self.prefill_budget = max(1, prefill_tokens)  # tokens per prefill pass
         self.cfg = model.cfg
+        self.vocab = getattr(model, "tp_vocab", model.cfg.vocab_size)  # whole vocabulary (a shard's cfg has its part)
         self.device = device or model.tok_emb.device
         self.max_batch = max_batch
         self.max_seq = min(max_seq, self.cfg.max_seq_len)
@@ -134,24 +123,13 @@ class Engine:
         self._pool = None
         self.scratch_slot = max_batch  # padding rows of a graphed step write here
         c = self.cfg
-        dt = model.tok_emb.dtype
         n_slots = max_batch + (1 if self.use_graphs else 0)
         if kv_pool_tokens is None and os.environ.get("MXLLM_KV_POOL_TOKENS"):
             kv_pool_tokens = int(os.environ["MXLLM_KV_POOL_TOKENS"])
-        from .kvcache import KVCache
+        from .steps import steps_for
 
-        self.kv = KVCache(c.n_layers, c.n_kv_heads, c.head_dim, dt, self.device, n_slots, self.max_seq,
-                          pool_tokens=kv_pool_tokens, block=kv_block,
-                          scratch_slot=self.scratch_slot if self.use_graphs else None)
-        # MXLLM_DECODE_COMBINE=fused: the split-K partials merge inside the attention launch (the
-        # last workgroup of each (seq, kv-head) combines; these counters stay zero between calls)
-        # instead of the combine kernel -- measured slower in the graphed step at every batch
-        # (archive/profiles/r3g/README.md), so off by default
-        self._attn_cnt = None
-        if self.device.type == "cuda" and os.environ.get("MXLLM_DECODE_COMBINE", "kernel") == "fused":
-            self._attn_cnt = torch.zeros((n_slots + 64) * self.kv.k[0].shape[1], dtype=torch.int32,
-                                         device=self.device)
-        self._pf_stream = torch.cuda.Stream(self.device) if self.device.type == "cuda" and _PREFETCH else None
+        self.model_steps = steps_for(model)(self)
+        self.kv = self.model_steps.make_cache(n_slots, kv_pool_tokens, kv_block)
         self.eos_ids = tuple(eos_ids) if eos_ids else (c.eos_id,)
         self.free_slots = list(range(max_batch))
         self.active: dict[int, Request] = {}
@@ -175,61 +153,6 @@ class Engine:
         self.latency_sum = 0.0
         self.finished = 0
 
-    # ------------------------------------------------------------------ model pieces
-    def _norm_proj(self, delta, h, gamma, lin, swiglu: bool):
-        """(proj(rmsnorm(h + delta) * gamma), h + delta); ``swiglu``: proj = swiglu(lin(.)).
-        Decode rows of a plain bf16 projection run as ONE launch (RMSNorm in the GEMM
-        prologue, SwiGLU in its epilogue: csrc/kernels/skinny_gemm.hip)."""
-        eps = self.cfg.norm_eps
-        plain = type(lin) is FusedLinear and lin.lora_r == 0
-        if _NORM_FUSED and plain:
-            r = ops.norm_linear(delta, h, gamma, eps, lin.weight, swiglu)
-            if r is not None:
-                return r
-        if delta is None:
-            xn = ops.rms_norm(h, gamma, eps)
-        else:
-            xn, h = ops.add_rms_norm(delta, h, gamma, eps)
-        if not swiglu:
-            return lin(xn), h
-        mid = None
-        if _SWIGLU_FUSED and plain and xn.dim() == 2:
-            mid = ops.linear_swiglu(xn, lin.weight)  # decode rows: SwiGLU in the GEMM epilogue
-        if mid is None:
-            mid = ops.swiglu(lin(xn))
-        return mid, h
-
-    @torch.no_grad()
-    def _layers(self, x: torch.Tensor, attn_fn, qkv_fn=None) -> torch.Tensor:
-        """``qkv_fn(i, delta, h, gamma, layer)`` (decode): the fused norm + QKV + RoPE/cache-append
-        projection returning (rotated q, new residual) or None; ``attn_fn(i, qkv, q=None)``."""
-        m, c = self.model, self.cfg
-        h = x
-        delta, gamma = None, m.layers[0].attn_norm  # sub-block output not yet added to h, next norm
-        for i, layer in enumerate(m.layers):
-            r = qkv_fn(i, delta, h, gamma, layer) if qkv_fn is not None else None
-            if r is not None:
-                q, h = r
-                o = attn_fn(i, None, q)
-            else:
-                qkv, h = self._norm_proj(delta, h, gamma, layer.wqkv, False)
-                o = attn_fn(i, qkv)
-            if isinstance(o, tuple):  # split-K partials: merged in the o-projection's prologue
-                a = ops.native().skinny_merge_linear(o[0], o[1], layer.wo.weight)
-            else:
-                a = layer.wo(o)
-            if self.tp is not None:  # row-parallel Wo: sum the heads' partial outputs
-                self.tp.all_reduce_(a)
-            mid, h = self._norm_proj(a, h, layer.mlp_norm, layer.wgu, True)
-            d = layer.wd(mid)
-            if self.tp is not None:  # row-parallel Wdown
-                self.tp.all_reduce_(d)
-            delta, gamma = d, (m.layers[i + 1].attn_norm if i + 1 < len(m.layers) else m.final_norm)
-        if delta is None:
-            return ops.rms_norm(h, gamma, c.norm_eps)
-        xn, h = ops.add_rms_norm(delta, h, gamma, c.norm_eps)
-        return xn
-
     @property
     def k_cache(self):
         return self.kv.k
@@ -244,6 +167,13 @@ class Engine:
         admission; direct ``prefill`` / ``decode`` callers may reserve themselves."""
         self.kv.reserve(slot, tokens)
 
+    def extend(self, slot: int, tokens: int) -> None:
+        """Let ``slot`` hold ``tokens`` positions, keeping what it holds (callers that decode without
+        knowing the final length)."""
+        if tokens > self.max_seq:
+            raise ValueError(f"{tokens} positions exceed max_seq {self.max_seq}")
+        self.kv.grow(slot, tokens)
+
     def _ensure(self, slot: int, tokens: int) -> None:
         if self.kv.capacity(slot) < tokens:
             if self.kv.paged and not self.kv.owned.get(slot):
@@ -255,21 +185,7 @@ class Engine:
     def prefill(self, slot: int, ids: list[int]) -> torch.Tensor:
         """Run the prompt through the model, filling ``slot``'s cache; returns
         last-position logits [V] (f32)."""
-        m, c = self.model, self.cfg
-        S = len(ids)
-        if S >= self.max_seq:
-            raise ValueError(f"prompt of {S} tokens exceeds max_seq {self.max_seq}")
-        self._ensure(slot, S + 1)
-        t = torch.tensor(ids, dtype=torch.long, device=self.device)
-        x = ops.embedding(t, m.tok_emb)
-
-        def attn(i, qkv):
-            return dops.prefill_attention(qkv, m.rope_cos, m.rope_sin, lambda k, v: self.kv.write(i, slot, k, v),
-                                          S, c.n_heads, c.n_kv_heads, c.head_dim)
-
-        xn = self._layers(x, attn)
-        self.lens[slot] = S
-        return self._logits(xn[-1:]).float()[0]
+        return self.prefill_batch([slot], [ids])[0]
 
     def _logits(self, xn: torch.Tensor) -> torch.Tensor:
         out = ops.linear(xn, self.model.head_weight)  # decode rows: the weight-streaming HIP GEMM
@@ -278,35 +194,30 @@ class Engine:
         return out
 
     @torch.no_grad()
-    def prefill_batch(self, slots: list[int], prompts: list[list[int]]) -> torch.Tensor:
+    def prefill_batch(self, slots: list[int], prompts: list[list[int]],
+                      want: list[list[int]] | None = None) -> torch.Tensor:
         """Prefill several prompts in ONE pass: their tokens are concatenated so
-        every GEMM / norm / SwiGLU runs once over all of them (each weight is
-        read once per batch instead of once per prompt); attention runs per
-        sequence into its own cache slot.  Returns last-position logits [n, V] f32."""
-        m, c = self.model, self.cfg
+        every GEMM / norm / activation runs once over all of them (each weight is
+        read once per batch instead of once per prompt).  Returns f32 logits of each
+        prompt's last position [n, V], or of the positions in ``want`` (per prompt, in order)."""
         lens = [len(p) for p in prompts]
         if any(S >= self.max_seq for S in lens):
-            raise ValueError(f"prompt exceeds max_seq {self.max_seq}")
+            raise ValueError(f"prompt of {max(lens)} tokens exceeds max_seq {self.max_seq}")
+        if any(not p or min(p) < 0 or max(p) >= self.vocab for p in prompts):
+            raise ValueError("empty prompt, or a token id outside the vocabulary")
         for s_, S in zip(slots, lens):
             self._ensure(s_, S + 1)
-        t = torch.tensor([tok for p in prompts for tok in p], dtype=torch.long, device=self.device)
-        x = ops.embedding(t, m.tok_emb)
-        offs = [0]
-        for S in lens:
-            offs.append(offs[-1] + S)
-
-        def attn(i, qkv):
-            outs = [dops.prefill_attention(qkv[offs[j]:offs[j + 1]], m.rope_cos, m.rope_sin,
-                                           lambda k, v, j=j: self.kv.write(i, slots[j], k, v), lens[j], c.n_heads,
-                                           c.n_kv_heads, c.head_dim)
-                    for j in range(len(prompts))]
-            return outs[0] if len(outs) == 1 else torch.cat(outs, 0)
-
-        xn = self._layers(x, attn)
+        xn = self.model_steps.prefill_hidden(slots, prompts)
         for s_, S in zip(slots, lens):
             self.lens[s_] = S
-        last = torch.tensor([o - 1 for o in offs[1:]], device=self.device)
-        return self._logits(xn.index_select(0, last)).float()
+        if want is None:
+            want = [[S - 1] for S in lens]
+        offs = [sum(lens[:i]) for i in range(len(lens))]
+        sel = [o + p for o, w in zip(offs, want) for p in w]
+        if not sel:
+            return torch.empty(0, self.vocab, device=self.device)
+        rows = xn[sel[0]:sel[0] + 1] if len(sel) == 1 else xn.index_select(0, torch.tensor(sel, device=self.device))
+        return self._logits(rows).float()
 
     @torch.no_grad()
     def decode(self, slots: list[int], tokens: torch.Tensor) -> torch.Tensor:
@@ -321,86 +232,18 @@ class Engine:
             inp = torch.stack([tokens.to(self.device, torch.long),
                                torch.tensor([self.lens[s] for s in slots], device=self.device),
                                torch.tensor(slots, device=self.device)])
-            logits = self._decode_body(inp, max_len)
+            logits = self.model_steps.decode_logits(inp, max_len)
         for s in slots:
             self.lens[s] += 1
         return logits[:B]
-
-    def _decode_body(self, inp: torch.Tensor, max_len: int) -> torch.Tensor:
-        """inp int64 [3, B] = (token, position of the new token, cache slot)."""
-        m, c = self.model, self.cfg
-        pos = inp[1].to(torch.int32)
-        sl = inp[2].to(torch.int32)
-        x = ops.embedding(inp[0], m.tok_emb)
-
-        bt = self.kv.bt
-        B = inp.shape[1]
-        nsplit = (min(max_len, self.kv.maxb * self.kv.block) + 255) // 256
-        merge = _MERGE_FUSED and c.head_dim == 128 and B <= 4 and nsplit <= 16
-        cnt = self._attn_cnt
-        if cnt is not None and B * self.kv.k[0].shape[1] > cnt.numel():
-            cnt = None
-
-        pf = self._pf_stream if B <= PREFETCH_MAX_B else None
-
-        def attn(i, qkv, q=None):
-            if pf is None:
-                return attn_(i, qkv, q)
-            wo = getattr(m.layers[i].wo, "weight", None)
-            if wo is None or not wo.is_contiguous():
-                return attn_(i, qkv, q)
-            cur = torch.cuda.current_stream(self.device)
-            pf.wait_stream(cur)
-            with torch.cuda.stream(pf):
-                ops.native().prefetch(wo, 128)
-            out = attn_(i, qkv, q)
-            cur.wait_stream(pf)  # joins the side branch before the o-projection
-            return out
-
-        def attn_(i, qkv, q=None):
-            if q is not None:  # RoPE and the cache append already done by the QKV GEMM
-                wo = m.layers[i].wo
-                K = q.shape[1] * 128  # this rank's heads (tensor parallel: a shard)
-                if (merge and type(wo) is FusedLinear and wo.lora_r == 0 and wo.weight.shape[0] % 16 == 0
-                        and K % 512 == 0 and B * K <= 32768 and wo.weight.shape[1] == K):
-                    # partials only: the split merge runs in the o-projection's prologue
-                    return ops.native().decode_attn_partials(q, self.kv.k[i], self.kv.v[i], pos, sl, max_len,
-                                                             1.0 / math.sqrt(c.head_dim), 1, bt)
-                return ops.native().decode_attn(q, self.kv.k[i], self.kv.v[i], pos, sl, max_len,
-                                                1.0 / math.sqrt(c.head_dim), 1, bt, cnt)
-            return dops.decode_attention(qkv, m.rope_cos, m.rope_sin, self.kv.k[i], self.kv.v[i], pos, sl,
-                                         c.n_heads, c.n_kv_heads, c.head_dim, max_len, bt, cnt)
-
-        def qkv_fn(i, delta, h, gamma, layer):
-            # QKV GEMM with the RoPE/cache-append epilogue; 1-2 rows also with the RMSNorm prologue
-            # (one launch), more rows after the RMSNorm kernel
-            if not (_ROPE_FUSED and self.tp is None and c.head_dim == 128
-                    and type(layer.wqkv) is FusedLinear and layer.wqkv.lora_r == 0):
-                return None
-            rope = (layer.wqkv.weight, m.rope_cos, m.rope_sin, pos, sl, self.kv.k[i], self.kv.v[i],
-                    c.n_heads, c.n_kv_heads, bt)
-            if _NORM_FUSED:
-                r = ops.qkv_rope_linear(delta, h, gamma, c.norm_eps, *rope)
-                if r is not None:
-                    return r
-            if not ops.qkv_rope_ok(h, rope[0], rope[1], rope[2], rope[5], rope[6], rope[7], rope[8], False):
-                return None
-            if delta is None:
-                xn = ops.rms_norm(h, gamma, c.norm_eps)
-            else:
-                xn, h = ops.add_rms_norm(delta, h, gamma, c.norm_eps)
-            q, _ = ops.qkv_rope_linear(None, xn, None, c.norm_eps, *rope)
-            return q, h
-
-        xn = self._layers(x, attn, qkv_fn)
-        return self._logits(xn)
 
     def _buckets(self, B: int, max_len: int) -> tuple[int, int]:
         bb = 1
         while bb < B:
             bb *= 2
         bb = min(bb, self.max_batch)
-        ns, cap = (max_len + 255) // 256, (self.max_seq + 255) // 256
+        # keys a step can look back over: the whole sequence, or a bounded span of it
+        ns, cap = (min(max_len, self.kv.span) + 255) // 256, (self.kv.span + 255) // 256
         nb = 1
         while nb < ns:
             nb *= 2
@@ -432,13 +275,13 @@ class Engine:
         side.wait_stream(torch.cuda.current_stream(self.device))
         with torch.cuda.stream(side):
             for _ in range(2):  # library handles / workspace set up outside capture
-                self._decode_body(inp, kl)
+                self.model_steps.decode_logits(inp, kl)
         torch.cuda.current_stream(self.device).wait_stream(side)
         graph = torch.cuda.CUDAGraph()
         if self._pool is None:
             self._pool = torch.cuda.graph_pool_handle()
         with torch.cuda.graph(graph, pool=self._pool, capture_error_mode="thread_local"):
-            out = self._decode_body(inp, kl)
+            out = self.model_steps.decode_logits(inp, kl)
         host = torch.empty(3, bb, dtype=torch.long, pin_memory=True)
         self._graphs[(bb, kl)] = (inp, out, graph, host)
         log.debug("captured decode graph: batch %d, key bound %d", bb, kl)
@@ -456,8 +299,7 @@ class Engine:
                 raise ValueError("empty input")
             if len(ids) >= self.max_seq:
                 raise ValueError(f"input of {len(ids)} tokens exceeds max_seq {self.max_seq}")
-            t = torch.tensor([ids], dtype=torch.long, device=self.device)
-            h = self.model.hidden_states(t).float()  # [S, H], final RMSNorm applied (no KV cache touched)
+            h = self.model_steps.hidden(ids).float()  # [S, H], final norm applied (no cache touched)
             out.append(torch.nn.functional.normalize(h.mean(0), dim=0))
         return torch.stack(out).cpu()
 

@@ -1,4 +1,4 @@
-"""Paged KV cache for the serving engine.
+"""Paged KV cache and per-sequence state for the serving engine.
 
 Per layer, K and V are POOLS of fixed-size blocks ``[blocks, Hkv, block, D]``
 (bf16) and every sequence slot maps its token positions to pool blocks through
@@ -20,6 +20,13 @@ Two modes:
     concurrent requests than slots sized for the longest one.
 
 One spare slot with one block takes the padding rows of a graphed decode step.
+
+``span``: a model whose layers all look back over a bounded run of positions keeps position p at
+row p % (that layer's run); a slot then needs blocks for ``span`` (the longest run) positions
+only, however long its sequence grows.
+
+``StateCache`` holds what a slot keeps at a fixed size: recurrent state (f32) and the last inputs
+of short convolutions.
 """
 from __future__ import annotations
 
@@ -32,12 +39,16 @@ BLOCK = 256
 
 class KVCache:
     def __init__(self, n_layers: int, n_kv_heads: int, head_dim: int, dtype, device, n_slots: int, max_seq: int,
-                 pool_tokens: int | None = None, block: int = BLOCK, scratch_slot: int | None = None):
+                 pool_tokens: int | None = None, block: int = BLOCK, scratch_slot: int | None = None,
+                 shapes: list[tuple[int, int, int]] | None = None, span: int | None = None):
+        """``shapes``: (kv heads, key width, value width) of each layer where they differ (the other
+        size arguments are then unused)."""
         if block % 256:
             raise ValueError("KV block size must be a multiple of 256 tokens (the decode split)")
         self.block = block
         self.max_seq = max_seq
-        self.maxb = math.ceil(max_seq / block)
+        self.span = max_seq if span is None else max(1, min(max_seq, span))
+        self.maxb = math.ceil(self.span / block)
         self.n_slots = n_slots
         self.paged = pool_tokens is not None
         self.scratch_slot = scratch_slot
@@ -47,9 +58,10 @@ class KVCache:
             n_blocks = (n_slots - (1 if scratch_slot is not None else 0)) * self.maxb
         n_blocks += 1 if scratch_slot is not None else 0
         self.n_blocks = n_blocks
-        self.k = [torch.zeros(n_blocks, n_kv_heads, block, head_dim, dtype=dtype, device=device)
-                  for _ in range(n_layers)]
-        self.v = [torch.zeros_like(k) for k in self.k]
+        if shapes is None:
+            shapes = [(n_kv_heads, head_dim, head_dim)] * n_layers
+        self.k = [torch.zeros(n_blocks, h, block, w, dtype=dtype, device=device) for h, w, _ in shapes]
+        self.v = [torch.zeros(n_blocks, h, block, w, dtype=dtype, device=device) for h, _, w in shapes]
         self.bt_host = torch.zeros(n_slots, self.maxb, dtype=torch.int32)
         self.owned: dict[int, list[int]] = {}
         self.free: list[int] = []
@@ -69,7 +81,7 @@ class KVCache:
 
     # ------------------------------------------------------------------ accounting
     def blocks_for(self, tokens: int) -> int:
-        return math.ceil(max(1, min(tokens, self.max_seq)) / self.block)
+        return math.ceil(max(1, min(tokens, self.span)) / self.block)
 
     @property
     def free_blocks(self) -> int:
@@ -91,18 +103,35 @@ class KVCache:
         if n > len(self.free):
             raise RuntimeError(f"KV pool exhausted: need {n} blocks, {len(self.free)} free")
         blocks, self.free = self.free[:n], self.free[n:]
+        self._assign(slot, blocks)
+
+    def _assign(self, slot: int, blocks: list[int]) -> None:
         self.owned[slot] = blocks
+        n = len(blocks)
         row = torch.zeros(self.maxb, dtype=torch.int32)
         row[:n] = torch.tensor(blocks, dtype=torch.int32)
         row[n:] = blocks[-1]  # never read (lengths stay inside the reservation); keeps the table in range
         self.bt_host[slot] = row
         self.bt[slot].copy_(row.to(self.bt.device), non_blocking=False)
 
+    def grow(self, slot: int, tokens: int) -> None:
+        """Add blocks until ``slot`` holds positions [0, tokens); what it holds stays (paged mode)."""
+        if not self.paged or self.capacity(slot) >= tokens:
+            return
+        have = self.owned.get(slot, [])
+        n = self.blocks_for(tokens) - len(have)
+        if n > len(self.free):
+            raise RuntimeError(f"KV pool exhausted: need {n} blocks, {len(self.free)} free")
+        if n > 0:
+            blocks, self.free = self.free[:n], self.free[n:]
+            self._assign(slot, have + blocks)
+
     def capacity(self, slot: int) -> int:
         """Positions ``slot`` can hold."""
         if not self.paged:
             return self.max_seq
-        return min(len(self.owned.get(slot, ())) * self.block, self.max_seq)
+        n = len(self.owned.get(slot, ())) * self.block
+        return self.max_seq if n >= self.span else n
 
     def release(self, slot: int) -> None:
         if self.paged and slot in self.owned and slot != self.scratch_slot:
@@ -144,3 +173,16 @@ class KVCache:
 
     def nbytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.k + self.v)
+
+
+class StateCache:
+    """Fixed-size per-slot state.  ``rec``: f32 [slots, width] per recurrent layer; ``conv``: [slots,
+    taps, channels] in the activation type per convolved layer, the input of position p at p % taps.
+    A new sequence writes its state without reading the slot's old one, so slots need no clearing."""
+
+    def __init__(self, n_slots: int, widths: list[int], convs: list[tuple[int, int]], dtype, device):
+        self.rec = [torch.zeros(n_slots, w, dtype=torch.float32, device=device) for w in widths]
+        self.conv = [torch.zeros(n_slots, n, c, dtype=dtype, device=device) for n, c in convs]
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in self.rec + self.conv)

@@ -96,7 +96,7 @@ class W8Linear(nn.Module):
 
 @torch.no_grad()
 def quantize_model_fp8_(model) -> int:
-    """Replace every transformer projection (qkv, o, gate/up, down) of a Llama by
+    """Replace every projection of the model's layers (a Llama's qkv, o, gate/up, down) by
     a :class:`W8Linear` (LoRA adapters are merged first).  Embedding, norms and
     the LM head stay bf16.  Returns the number of weight bytes saved."""
     from ..models.llama import FusedLinear
@@ -105,8 +105,7 @@ def quantize_model_fp8_(model) -> int:
     merge_lora_(model)
     saved = 0
     for layer in model.layers:
-        for name in ("wqkv", "wo", "wgu", "wd"):
-            lin = getattr(layer, name)
+        for name, lin in list(layer.named_children()):
             if isinstance(lin, FusedLinear):
                 w = lin.weight
                 setattr(layer, name, W8Linear(w))

@@ -1,0 +1,255 @@
+"""The model-specific part of the serving engine: one steps object per model class.
+
+``Engine`` (mxllm/serve/engine.py) owns slots, scheduling, graphs and sampling; its steps object
+builds the caches and runs the layer stack:
+
+  * ``make_cache``     : the KVCache (and per-slot state) of the model, sized for the engine's slots;
+  * ``prefill_hidden`` : whole prompts -> final normed hidden rows of all their tokens, caches filled;
+  * ``decode_logits``  : one token per slot -> logits; graph-captured, so device work only;
+  * ``hidden``         : one sequence -> final normed hidden rows, nothing cached (embeddings).
+
+``STEPS`` maps a model class to its steps class; a new design adds an entry.
+"""
+from __future__ import annotations
+
+import math
+import os
+
+import torch
+
+from .. import ops
+from ..models.llama import FusedLinear, Llama
+from ..models.revesun import Revesun
+from ..ops import decode as dops
+from ..ops.hybrid import PromptRows, SeqCaches, TokenRows
+from .kvcache import KVCache, StateCache
+
+_SWIGLU_FUSED = os.environ.get("MXLLM_SWIGLU_FUSED", "1") != "0"  # A/B switch (bench/serve_bench.py)
+_NORM_FUSED = os.environ.get("MXLLM_NORM_FUSED", "1") != "0"  # A/B switch: RMSNorm in the decode GEMM prologue
+_ROPE_FUSED = os.environ.get("MXLLM_ROPE_FUSED", "1") != "0"  # A/B switch: RoPE + cache append in the QKV epilogue
+# the split-K attention merge in the o-projection GEMM's prologue (decode rows <= 4): OFF by
+# default -- measured 8B decode, same box: batch 1 3.424 vs 3.433 ms (a wash), batch 4 4.113 vs
+# 3.841 ms (the prologue slows the weight stream more than the combine launch costs;
+# archive/profiles/r3d_decode_merge_ab.md).  MXLLM_MERGE_FUSED=1 turns it on.
+_MERGE_FUSED = os.environ.get("MXLLM_MERGE_FUSED", "0") == "1"
+# Small-batch decode: while the (latency-bound) attention runs, a side-stream kernel reads
+# the layer's o-projection weight so the o-projection GEMM streams it from the Infinity
+# Cache instead of HBM (MXLLM_DECODE_PREFETCH=1; up to PREFETCH_MAX_B rows).  Measured
+# slower (fork/join + competing reads; archive/profiles/r3g/README.md): off by default.
+_PREFETCH = os.environ.get("MXLLM_DECODE_PREFETCH", "0") == "1"
+PREFETCH_MAX_B = 8
+
+
+class LlamaSteps:
+    def __init__(self, eng):
+        self.eng, self.model, self.cfg = eng, eng.model, eng.cfg
+
+    def make_cache(self, n_slots: int, pool_tokens: int | None, block: int) -> KVCache:
+        eng, c = self.eng, self.cfg
+        kv = KVCache(c.n_layers, c.n_kv_heads, c.head_dim, self.model.tok_emb.dtype, eng.device, n_slots, eng.max_seq,
+                     pool_tokens=pool_tokens, block=block,
+                     scratch_slot=eng.scratch_slot if eng.use_graphs else None)
+        # MXLLM_DECODE_COMBINE=fused: the split-K partials merge inside the attention launch (the
+        # last workgroup of each (seq, kv-head) combines; these counters stay zero between calls)
+        # instead of the combine kernel -- measured slower in the graphed step at every batch
+        # (archive/profiles/r3g/README.md), so off by default
+        eng._attn_cnt = None
+        if eng.device.type == "cuda" and os.environ.get("MXLLM_DECODE_COMBINE", "kernel") == "fused":
+            eng._attn_cnt = torch.zeros((n_slots + 64) * kv.k[0].shape[1], dtype=torch.int32,
+                                         device=eng.device)
+        eng._pf_stream = torch.cuda.Stream(eng.device) if eng.device.type == "cuda" and _PREFETCH else None
+        return kv
+
+    def hidden(self, ids: list[int]) -> torch.Tensor:
+        return self.model.hidden_states(torch.tensor([ids], dtype=torch.long, device=self.eng.device))
+
+    def prefill_hidden(self, slots: list[int], prompts: list[list[int]]) -> torch.Tensor:
+        """Concatenated tokens through the GEMMs; attention per sequence into its own cache slot."""
+        m, c, eng = self.model, self.cfg, self.eng
+        lens = [len(p) for p in prompts]
+        t = torch.tensor([tok for p in prompts for tok in p], dtype=torch.long, device=eng.device)
+        x = ops.embedding(t, m.tok_emb)
+        offs = [0]
+        for S in lens:
+            offs.append(offs[-1] + S)
+
+        def attn(i, qkv):
+            outs = [dops.prefill_attention(qkv[offs[j]:offs[j + 1]], m.rope_cos, m.rope_sin,
+                                           lambda k, v, j=j: eng.kv.write(i, slots[j], k, v), lens[j], c.n_heads,
+                                           c.n_kv_heads, c.head_dim)
+                    for j in range(len(prompts))]
+            return outs[0] if len(outs) == 1 else torch.cat(outs, 0)
+
+        return self._layers(x, attn)
+
+    def _norm_proj(self, delta, h, gamma, lin, swiglu: bool):
+        """(proj(rmsnorm(h + delta) * gamma), h + delta); ``swiglu``: proj = swiglu(lin(.)).
+        Decode rows of a plain bf16 projection run as ONE launch (RMSNorm in the GEMM
+        prologue, SwiGLU in its epilogue: csrc/kernels/skinny_gemm.hip)."""
+        eps = self.cfg.norm_eps
+        plain = type(lin) is FusedLinear and lin.lora_r == 0
+        if _NORM_FUSED and plain:
+            r = ops.norm_linear(delta, h, gamma, eps, lin.weight, swiglu)
+            if r is not None:
+                return r
+        if delta is None:
+            xn = ops.rms_norm(h, gamma, eps)
+        else:
+            xn, h = ops.add_rms_norm(delta, h, gamma, eps)
+        if not swiglu:
+            return lin(xn), h
+        mid = None
+        if _SWIGLU_FUSED and plain and xn.dim() == 2:
+            mid = ops.linear_swiglu(xn, lin.weight)  # decode rows: SwiGLU in the GEMM epilogue
+        if mid is None:
+            mid = ops.swiglu(lin(xn))
+        return mid, h
+
+    @torch.no_grad()
+    def _layers(self, x: torch.Tensor, attn_fn, qkv_fn=None) -> torch.Tensor:
+        """``qkv_fn(i, delta, h, gamma, layer)`` (decode): the fused norm + QKV + RoPE/cache-append
+        projection returning (rotated q, new residual) or None; ``attn_fn(i, qkv, q=None)``."""
+        m, c = self.model, self.cfg
+        tp = self.eng.tp
+        h = x
+        delta, gamma = None, m.layers[0].attn_norm  # sub-block output not yet added to h, next norm
+        for i, layer in enumerate(m.layers):
+            r = qkv_fn(i, delta, h, gamma, layer) if qkv_fn is not None else None
+            if r is not None:
+                q, h = r
+                o = attn_fn(i, None, q)
+            else:
+                qkv, h = self._norm_proj(delta, h, gamma, layer.wqkv, False)
+                o = attn_fn(i, qkv)
+            if isinstance(o, tuple):  # split-K partials: merged in the o-projection's prologue
+                a = ops.native().skinny_merge_linear(o[0], o[1], layer.wo.weight)
+            else:
+                a = layer.wo(o)
+            if tp is not None:  # row-parallel Wo: sum the heads' partial outputs
+                tp.all_reduce_(a)
+            mid, h = self._norm_proj(a, h, layer.mlp_norm, layer.wgu, True)
+            d = layer.wd(mid)
+            if tp is not None:  # row-parallel Wdown
+                tp.all_reduce_(d)
+            delta, gamma = d, (m.layers[i + 1].attn_norm if i + 1 < len(m.layers) else m.final_norm)
+        if delta is None:
+            return ops.rms_norm(h, gamma, c.norm_eps)
+        xn, h = ops.add_rms_norm(delta, h, gamma, c.norm_eps)
+        return xn
+
+    def decode_logits(self, inp: torch.Tensor, max_len: int) -> torch.Tensor:
+        """inp int64 [3, B] = (token, position of the new token, cache slot)."""
+        m, c = self.model, self.cfg
+        pos = inp[1].to(torch.int32)
+        sl = inp[2].to(torch.int32)
+        x = ops.embedding(inp[0], m.tok_emb)
+
+        bt = self.eng.kv.bt
+        B = inp.shape[1]
+        nsplit = (min(max_len, self.eng.kv.maxb * self.eng.kv.block) + 255) // 256
+        merge = _MERGE_FUSED and c.head_dim == 128 and B <= 4 and nsplit <= 16
+        cnt = self.eng._attn_cnt
+        if cnt is not None and B * self.eng.kv.k[0].shape[1] > cnt.numel():
+            cnt = None
+
+        pf = self.eng._pf_stream if B <= PREFETCH_MAX_B else None
+
+        def attn(i, qkv, q=None):
+            if pf is None:
+                return attn_(i, qkv, q)
+            wo = getattr(m.layers[i].wo, "weight", None)
+            if wo is None or not wo.is_contiguous():
+                return attn_(i, qkv, q)
+            cur = torch.cuda.current_stream(self.eng.device)
+            pf.wait_stream(cur)
+            with torch.cuda.stream(pf):
+                ops.native().prefetch(wo, 128)
+            out = attn_(i, qkv, q)
+            cur.wait_stream(pf)  # joins the side branch before the o-projection
+            return out
+
+        def attn_(i, qkv, q=None):
+            if q is not None:  # RoPE and the cache append already done by the QKV GEMM
+                wo = m.layers[i].wo
+                K = q.shape[1] * 128  # this rank's heads (tensor parallel: a shard)
+                if (merge and type(wo) is FusedLinear and wo.lora_r == 0 and wo.weight.shape[0] % 16 == 0
+                        and K % 512 == 0 and B * K <= 32768 and wo.weight.shape[1] == K):
+                    # partials only: the split merge runs in the o-projection's prologue
+                    return ops.native().decode_attn_partials(q, self.eng.kv.k[i], self.eng.kv.v[i], pos, sl, max_len,
+                                                             1.0 / math.sqrt(c.head_dim), 1, bt)
+                return ops.native().decode_attn(q, self.eng.kv.k[i], self.eng.kv.v[i], pos, sl, max_len,
+                                                1.0 / math.sqrt(c.head_dim), 1, bt, cnt)
+            return dops.decode_attention(qkv, m.rope_cos, m.rope_sin, self.eng.kv.k[i], self.eng.kv.v[i], pos, sl,
+                                         c.n_heads, c.n_kv_heads, c.head_dim, max_len, bt, cnt)
+
+        def qkv_fn(i, delta, h, gamma, layer):
+            # QKV GEMM with the RoPE/cache-append epilogue; 1-2 rows also with the RMSNorm prologue
+            # (one launch), more rows after the RMSNorm kernel
+            if not (_ROPE_FUSED and self.eng.tp is None and c.head_dim == 128
+                    and type(layer.wqkv) is FusedLinear and layer.wqkv.lora_r == 0):
+                return None
+            rope = (layer.wqkv.weight, m.rope_cos, m.rope_sin, pos, sl, self.eng.kv.k[i], self.eng.kv.v[i],
+                    c.n_heads, c.n_kv_heads, bt)
+            if _NORM_FUSED:
+                r = ops.qkv_rope_linear(delta, h, gamma, c.norm_eps, *rope)
+                if r is not None:
+                    return r
+            if not ops.qkv_rope_ok(h, rope[0], rope[1], rope[2], rope[5], rope[6], rope[7], rope[8], False):
+                return None
+            if delta is None:
+                xn = ops.rms_norm(h, gamma, c.norm_eps)
+            else:
+                xn, h = ops.add_rms_norm(delta, h, gamma, c.norm_eps)
+            q, _ = ops.qkv_rope_linear(None, xn, None, c.norm_eps, *rope)
+            return q, h
+
+        xn = self._layers(x, attn, qkv_fn)
+        return self.eng._logits(xn)
+
+
+class RevesunSteps:
+    """Attention layers keep the current chunk's keys and the convolution's last inputs, recurrent
+    layers an f32 state; the layer stack itself is ``Revesun.rows``."""
+
+    def __init__(self, eng):
+        if eng.tp is not None:
+            raise NotImplementedError("Revesun is served on one GPU (no tensor-parallel sharding)")
+        self.eng, self.model, self.cfg = eng, eng.model, eng.cfg
+
+    def make_cache(self, n_slots: int, pool_tokens: int | None, block: int) -> KVCache:
+        eng, dt = self.eng, self.model.dtype
+        attn = [s.attn for s in self.cfg.layers if s.kind == "attention"]
+        self.kv = KVCache(len(attn), 0, 0, dt, eng.device, n_slots, eng.max_seq, pool_tokens=pool_tokens, block=block,
+                          scratch_slot=eng.scratch_slot if eng.use_graphs else None,
+                          shapes=[(a.kv_heads, *a.row_dims(dt)) for a in attn],
+                          span=max((a.chunk for a in attn), default=1))
+        self.state = StateCache(n_slots, [s.width for s in self.cfg.layers if s.kind == "mingru"],
+                                [(a.taps, a.conv_channels) for a in attn], dt, eng.device)
+        self.caches = SeqCaches(self.kv.k, self.kv.v, self.kv.bt, self.state.conv, self.state.rec)
+        self.model.prepare(eng.max_seq)
+        return self.kv
+
+    def _ids(self, prompts: list[list[int]]) -> torch.Tensor:
+        return torch.tensor([tok for p in prompts for tok in p], dtype=torch.long).to(self.eng.device)
+
+    def hidden(self, ids: list[int]) -> torch.Tensor:
+        return self.model.rows(self._ids([ids]), PromptRows([len(ids)], self.eng.device))
+
+    def prefill_hidden(self, slots: list[int], prompts: list[list[int]]) -> torch.Tensor:
+        rows = PromptRows([len(p) for p in prompts], self.eng.device, slots, self.caches)
+        return self.model.rows(self._ids(prompts), rows)
+
+    def decode_logits(self, inp: torch.Tensor, max_len: int) -> torch.Tensor:
+        """inp int64 [3, B] = (token, position of the new token, cache slot)."""
+        pos, sl = inp[1:].to(torch.int32)
+        return self.eng._logits(self.model.rows(inp[0], TokenRows(pos, sl, max_len, self.caches)))
+
+
+STEPS = {Llama: LlamaSteps, Revesun: RevesunSteps}
+
+
+def steps_for(model) -> type:
+    for cls in type(model).__mro__:
+        if cls in STEPS:
+            return STEPS[cls]
+    return LlamaSteps  # Llama-shaped shards (mxllm/parallel/tensor.py)

@@ -169,7 +169,7 @@ def test_engine_in_launch_decode_merge_matches_combine_kernel(gpu, monkeypatch):
 def test_engine_decode_prefetch_is_transparent(gpu, monkeypatch):
     """MXLLM_DECODE_PREFETCH=1 (a side-stream read of each o-projection weight during the
     decode attention, joined before the GEMM, captured into the decode graph) changes no token."""
-    import mxllm.serve.engine as E
+    import mxllm.serve.steps as E
 
     m = Llama(get_config("tiny-d128"), device=gpu, seed=5).eval()
     prompts = [list(range(1 + i, 60 + 31 * i)) for i in range(3)]
