@@ -1,6 +1,7 @@
 """``python -m mxllm <command>`` (also the ``mxllm`` console script).
 
   serve      OpenAI-compatible server (mxllm.serve.server; same flags)
+  trace      replay a token trace through the engine and write logits (mxllm.serve.trace; bin/trace_run)
   build      compile the gfx950 native library (mxllm._build; same flags)
   export-hf  a trained model as a Hugging Face Llama directory: base weights (a preset with
              its seed, or an HF directory) + the weights an mxllm run saved (a checkpoint
@@ -67,6 +68,10 @@ def main(argv=None) -> int:
 
         serve_main(rest)
         return 0
+    if cmd == "trace":
+        from .serve.trace import main as trace_main
+
+        return trace_main(rest)
     if cmd == "build":
         from ._build import main as build_main
 

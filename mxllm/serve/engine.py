@@ -167,6 +167,17 @@ class Engine:
         admission; direct ``prefill`` / ``decode`` callers may reserve themselves."""
         self.kv.reserve(slot, tokens)
 
+    def acquire(self) -> int:
+        """A free slot, for callers that run prefill / decode themselves (give it back with release)."""
+        if not self.free_slots:
+            raise RuntimeError(f"all {self.max_batch} sequence slots are in use")
+        return self.free_slots.pop(0)
+
+    def release(self, slot: int) -> None:
+        self.kv.release(slot)
+        self.lens[slot] = 0
+        self.free_slots.append(slot)
+
     def extend(self, slot: int, tokens: int) -> None:
         """Let ``slot`` hold ``tokens`` positions, keeping what it holds (callers that decode without
         knowing the final length)."""

@@ -14,6 +14,7 @@ from __future__ import annotations
 
 import math
 import os
+import weakref
 
 import torch
 
@@ -42,7 +43,7 @@ PREFETCH_MAX_B = 8
 
 class LlamaSteps:
     def __init__(self, eng):
-        self.eng, self.model, self.cfg = eng, eng.model, eng.cfg
+        self.eng, self.model, self.cfg = weakref.proxy(eng), eng.model, eng.cfg  # no cycle: caches go with the engine
 
     def make_cache(self, n_slots: int, pool_tokens: int | None, block: int) -> KVCache:
         eng, c = self.eng, self.cfg
@@ -214,7 +215,7 @@ class RevesunSteps:
     def __init__(self, eng):
         if eng.tp is not None:
             raise NotImplementedError("Revesun is served on one GPU (no tensor-parallel sharding)")
-        self.eng, self.model, self.cfg = eng, eng.model, eng.cfg
+        self.eng, self.model, self.cfg = weakref.proxy(eng), eng.model, eng.cfg  # no cycle: caches go with the engine
 
     def make_cache(self, n_slots: int, pool_tokens: int | None, block: int) -> KVCache:
         eng, dt = self.eng, self.model.dtype
