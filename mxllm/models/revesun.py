@@ -159,6 +159,7 @@ class Revesun(nn.Module):
             self.kind_index.append(count[s.kind])
             count[s.kind] += 1
         self._rope: dict = {}
+        self._rope_kept: list = []
         if init:
             self.reset_parameters(seed)
         self.requires_grad_(False)
@@ -191,6 +192,7 @@ class Revesun(nn.Module):
         have = self._rope.get(key)
         if have is None or have[0].shape[0] < n:
             n = max(n, 256)
+            self._rope_kept.append(have)  # captured decode graphs may still read the shorter tables
             have = hops.pair_rope_tables(n, *key, device=self.tok_emb.device)
             self._rope[key] = have
         return have
@@ -208,7 +210,7 @@ class Revesun(nn.Module):
     def rows(self, ids: torch.Tensor, rows, tap=None) -> torch.Tensor:
         """Final normed hidden rows of token ``ids`` [T] laid out as ``rows``.  ``tap(i, h)``: the
         residual stream after layer i (diagnostics)."""
-        n = rows.max_len if rows.decode else max(rows.lens)
+        n = 0 if rows.decode else max(rows.lens)  # decode: the tables prepare() sized
         h = hops.embed_rows(ids, self.tok_emb)
         delta = None
         for i, layer in enumerate(self.layers):
@@ -324,7 +326,7 @@ def _stack(n: int, width: int, heads: int, kv: int, dim: int, chunk: int, ff: in
 PRESETS["revesun-tiny"] = RevesunConfig("revesun-tiny", 320, 64, _stack(4, 96, 4, 2, 16, 24, 160, 1e4), norm_groups=2)
 # projection and feed-forward sizes of the Llama presets of the same name (two feed-forward matrices of
 # 1.5x the width in place of three)
-PRESETS["revesun-1b"] = RevesunConfig("revesun-1b", 128256, 2048, _stack(16, 2048, 16, 4, 128, 4096, 12288, 5e5),
+PRESETS["revesun-1b"] = RevesunConfig("revesun-1b", 128256, 2048, _stack(16, 2048, 32, 8, 64, 4096, 12288, 5e5),
                                       norm_groups=8)
 PRESETS["revesun-8b"] = RevesunConfig("revesun-8b", 128256, 4096, _stack(32, 4096, 32, 8, 128, 4096, 21504, 5e5),
                                       norm_groups=8)

@@ -132,7 +132,7 @@ class PromptRows:
 
 class TokenRows:
     """One token per sequence: ``pos`` / ``slots`` int32 [B] on the device, ``max_len`` a host bound
-    on pos + 1."""
+    on the keys a step looks back over (pos + 1, or the longest chunk)."""
 
     decode = True
 
@@ -142,8 +142,6 @@ class TokenRows:
 
     def chunk_pos(self, chunk: int) -> torch.Tensor:
         """Position inside the chunk = index of the newest cached row."""
-        if chunk >= self.max_len:
-            return self.pos
         if chunk not in self._local:
             self._local[chunk] = torch.remainder(self.pos, chunk)
         return self._local[chunk]

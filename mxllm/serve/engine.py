@@ -266,9 +266,10 @@ class Engine:
         entry = self._graphs.get((bb, kl))
         if entry is None:
             entry = self._capture(bb, kl)
-        inp, out, graph, host = entry
-        # the previous step's copy from ``host`` has completed: its logits were
-        # read back (sampling) before this step was scheduled
+        inp, out, graph, host, copied = entry
+        # the previous step's copy from ``host`` must have completed (it has where the caller
+        # read that step's logits back, as sampling does)
+        copied.synchronize()
         host[0, :B] = tokens.to("cpu", torch.long)
         host[1, :B] = torch.tensor([self.lens[s] for s in slots])
         host[2, :B] = torch.tensor(slots)
@@ -276,6 +277,7 @@ class Engine:
         host[1, B:] = 0
         host[2, B:] = self.scratch_slot
         inp.copy_(host, non_blocking=True)
+        copied.record()
         graph.replay()
         return out
 
@@ -294,7 +296,7 @@ class Engine:
         with torch.cuda.graph(graph, pool=self._pool, capture_error_mode="thread_local"):
             out = self.model_steps.decode_logits(inp, kl)
         host = torch.empty(3, bb, dtype=torch.long, pin_memory=True)
-        self._graphs[(bb, kl)] = (inp, out, graph, host)
+        self._graphs[(bb, kl)] = (inp, out, graph, host, torch.cuda.Event())
         log.debug("captured decode graph: batch %d, key bound %d", bb, kl)
         return self._graphs[(bb, kl)]
 
