@@ -27,6 +27,10 @@ in a fresh 8-rank child job, and reported under ``config4_full_zero3`` in the
 same JSON line.  ``--emulate-world N`` runs ZeRO-3 in one process with world-N
 shard sizes (per-rank memory/compute proxy without link traffic).
 
+``--serve MODEL[,MODEL...]`` measures serving instead (bench/serve_bench.py: prefill tokens/s, graphed decode
+step at several batches) for the named presets one after the other and prints one JSON line; everything
+above stays as it is without it.
+
 ``--gpus N`` without a torchrun environment spawns the N ranks itself (child
 ``torch.distributed.run``, rendezvous on 127.0.0.1); under torchrun a
 WORLD_SIZE different from N is an error (exit 1).
@@ -75,6 +79,11 @@ def parse(argv=None):
     ap.add_argument("--device", default=None, help="force 'cpu' for a plumbing run")
     ap.add_argument("--layers", type=int, default=None, help="override n_layers (NOT valid for the headline)")
     ap.add_argument("--json-out", default=None)
+    ap.add_argument("--serve", default="", metavar="MODELS",
+                    help="serving throughput of these presets (comma list, e.g. revesun-8b,llama3.1-8b) instead of training")
+    ap.add_argument("--serve-prompt-len", type=int, default=4096)
+    ap.add_argument("--serve-ctx", type=int, default=2048, help="cached tokens per sequence in the decode sweep")
+    ap.add_argument("--serve-batches", default="1,4,8,32")
     ap.add_argument("--no-gemm-table", action="store_true", help="ignore the tuned hipBLASLt solution table")
     ap.add_argument("--emulate-world", type=int, default=0,
                     help="zero3 only: one process holding world-N shard sizes (gathers tile the local shard)")
@@ -233,6 +242,8 @@ def check_world(gpus: int) -> str:
 def main(argv=None):
     argv = list(sys.argv[1:] if argv is None else argv)
     a = parse(argv)
+    if a.serve:
+        return run_serve(a)
     mode = check_world(a.gpus)
     if mode == "mismatch":
         print(f"bench.py: --gpus {a.gpus} but the launcher started WORLD_SIZE={os.environ['WORLD_SIZE']} ranks",
@@ -325,6 +336,31 @@ def main(argv=None):
         if env.is_main:
             _emit_once()
         runtime.cleanup()
+
+
+def run_serve(a) -> int:
+    """``--serve``: prefill and decode throughput of the named presets, one JSON line."""
+    import contextlib
+    import gc
+
+    sys.path.insert(0, os.path.join(ROOT, "bench"))
+    from serve_bench import main as serve_main
+
+    rows = []
+    for model in a.serve.split(","):
+        print(f"[bench] serving {model}", file=sys.stderr, flush=True)
+        with contextlib.redirect_stdout(sys.stderr):
+            rows.append(serve_main(["--model", model, "--prompt-len", str(a.serve_prompt_len), "--ctx",
+                                    str(a.serve_ctx), "--batches", a.serve_batches, "--requests", "0"]))
+        gc.collect()
+        torch.cuda.empty_cache()
+    line = json.dumps({"metric": "serving throughput (prefill, decode)", "dtype": "bf16",
+                       "data": "synthetic prompts, random-init weights", "models": rows})
+    print(line, flush=True)
+    if a.json_out:
+        with open(a.json_out, "w") as f:
+            f.write(line + "\n")
+    return 0
 
 
 def _arm_emit_on_signal(out: dict, json_out: str | None) -> None:

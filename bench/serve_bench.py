@@ -33,7 +33,7 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 sys.path.insert(0, ROOT)
 
 
-def main():
+def main(argv=None) -> dict:
     ap = argparse.ArgumentParser()
     ap.add_argument("--model", default="llama3.1-8b")
     ap.add_argument("--prompt-len", type=int, default=1024)
@@ -51,9 +51,9 @@ def main():
                     help="paged KV cache shared by all slots (default: every slot owns max_seq positions)")
     ap.add_argument("--tp-shard-proxy", type=int, default=0,
                     help="one GPU: run rank 0's TP-N shard without the collectives (per-GPU compute floor)")
-    a = ap.parse_args()
+    a = ap.parse_args(argv)
 
-    from mxllm.models import Llama, get_config
+    from mxllm.models import build_model, get_config
     from mxllm.serve.engine import Engine
     from mxllm.utils import gemm_tuning
 
@@ -78,7 +78,7 @@ def main():
 
         model = random_shard(cfg, rank, tp, dev, seed=0)
     else:
-        model = Llama(cfg, device=dev, dtype=torch.bfloat16, seed=0)
+        model = build_model(a.model, device=dev, dtype=torch.bfloat16, seed=0)
     model.requires_grad_(False)
     full_cfg, cfg = cfg, model.cfg  # per-rank shapes from here on (KV bytes, prompts use the vocab below)
     if a.fp8:
@@ -92,6 +92,7 @@ def main():
     bmax = max(int(b) for b in a.batches.split(","))
     max_seq = max(a.prompt_len, a.ctx + a.decode_steps, a.e2e_prompt_len + a.new_tokens) + 8
     eng = Engine(model, max_batch=max(bmax, 1), max_seq=max_seq, tp_group=tp_group, kv_pool_tokens=a.kv_pool_tokens)
+    chunks = [s.attn.chunk for s in cfg.layers if s.kind == "attention"] if hasattr(cfg, "layers") else [0] * cfg.n_layers
     g = torch.Generator().manual_seed(0)
 
     def prompt(n):
@@ -135,7 +136,10 @@ def main():
             eng.decode(slots, tok)
         torch.cuda.synchronize()
         dt = (time.perf_counter() - t) / a.decode_steps
-        kv_bytes = bs * (a.ctx + a.decode_steps // 2) * cfg.n_layers * 2 * cfg.n_kv_heads * cfg.head_dim * 2
+        # cached rows a step reads: a layer looks back over its chunk of positions, or over all of them
+        kv_bytes = bs * sum((c.shape[1] * c.shape[3] * c.element_size())
+                            * ((a.ctx + a.decode_steps // 2) % chunk if chunk else a.ctx + a.decode_steps // 2)
+                            for pool in (eng.kv.k, eng.kv.v) for c, chunk in zip(pool, chunks))
         out["decode"].append({"batch": bs, "ctx": a.ctx, "ms_per_step": round(1e3 * dt, 3),
                               "tokens_per_s": round(bs / dt, 1),
                               "weight_stream_tb_s": round(wbytes / dt / 1e12, 2),
@@ -186,6 +190,7 @@ def main():
                 f.write(line + "\n")
     if world > 1:
         runtime.cleanup()
+    return out
 
 
 if __name__ == "__main__":

@@ -50,14 +50,14 @@ def main():
     ap.add_argument("--prefill", default="", help="also tune the prefill GEMMs of these prompt lengths (e.g. 1024)")
     a = ap.parse_args()
 
-    from mxllm.models import Llama, get_config
+    from mxllm.models import build_model, get_config
     from mxllm.serve.engine import Engine
     from mxllm.utils import gemm_tuning
 
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
     cfg = get_config(a.model)
-    model = Llama(cfg, device=dev, dtype=torch.bfloat16, seed=0)
+    model = build_model(a.model, device=dev, dtype=torch.bfloat16, seed=0)
     model.requires_grad_(False)
     batches = [int(b) for b in a.batches.split(",")]
     plens = [int(x) for x in a.prefill.split(",") if x]

@@ -146,8 +146,7 @@ int mx_lora_xtg(const int64_t* desc, int np, int T, float alpha, int accumulate,
 int mx_embed_rows(const int64_t* ids, const void* w, int f32, float* out, int64_t T, int W, int V, hipStream_t stream);
 int mx_group_norm(const void* delta, int64_t ldd, float* h, const float* w, void* y, int64_t ldy, int f32, int64_t T,
                   int W, int groups, float eps, hipStream_t stream);
-int mx_conv_rope_prefill(const mx::ConvRope* a, int f32, const int32_t* rowpos, const int32_t* rowseq,
-                         const int32_t* seqs, int T, hipStream_t stream);
+int mx_conv_rope_prefill(const mx::ConvRope* a, int f32, const int32_t* rows, int T, hipStream_t stream);
 int mx_conv_rope_decode(const mx::ConvRope* a, int f32, const int32_t* pos, const int32_t* slots, int B,
                         hipStream_t stream);
 int mx_poly_norm(const void* z, int64_t ldz, const float* coef, void* y, int f32, int64_t T, int F, float eps,
@@ -166,4 +165,18 @@ int mx_mingru_scan(const void* x, int64_t ldx, int f32, const float* bias, const
                    hipStream_t stream);
 int mx_mingru_step(const void* x, int64_t ldx, int f32, const float* bias, const int32_t* slots, float* state, void* y,
                    int B, int W, hipStream_t stream);
+// hybrid_skinny.hip
+int mx_hs_norm_gemm(const uint16_t* delta, int64_t ldd, const float* h, const float* gamma, float* h_out, int groups,
+                    float eps, const uint16_t* w, int64_t ldw, uint16_t* y, int64_t ldy, int M, int N, int K,
+                    hipStream_t stream);
+int mx_hs_poly_gemm(const uint16_t* z, int64_t ldz, const float* coef, float eps, const uint16_t* w, int64_t ldw,
+                    uint16_t* y, int64_t ldy, int M, int N, int K, hipStream_t stream);
+int mx_hs_gru_gemm(const uint16_t* x, int64_t ldx, int norm, const uint16_t* delta, int64_t ldd, const float* h,
+                   const float* gamma, float* h_out, int groups, float eps, const uint16_t* w, int64_t ldw,
+                   const float* bias, const int32_t* slots, float* state, uint16_t* y, int M, int W, int K,
+                   hipStream_t stream);
+int mx_hs_conv_gemm(const uint16_t* x, int64_t ldx, int norm, const uint16_t* delta, int64_t ldd, const float* h,
+                    const float* gamma, float* h_out, int groups, float eps, const uint16_t* w, int64_t ldw,
+                    const mx::ConvRope* a, const int32_t* pos, const int32_t* slots, uint16_t* gate, int M, int K,
+                    hipStream_t stream);
 }

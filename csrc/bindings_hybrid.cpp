@@ -62,6 +62,83 @@ at::Tensor group_norm(const c10::optional<at::Tensor>& delta, at::Tensor h, cons
   return y;
 }
 
+// ---- fused decode GEMMs (hybrid_skinny.hip): bf16 rows, weights [N, K] with unit inner stride
+struct HsIn {  // X = x, or group_norm(h + delta) * gamma with the new residual in h_out
+  const uint16_t *x = nullptr, *delta = nullptr;
+  const float *h = nullptr, *gamma = nullptr;
+  float* h_out = nullptr;
+  int64_t ldx = 0, ldd = 0, M = 0, K = 0;
+  int norm = 0;
+  at::Tensor hn;
+};
+HsIn hs_in(const at::Tensor& x, const c10::optional<at::Tensor>& delta, const c10::optional<at::Tensor>& gamma,
+           const at::Tensor& w) {
+  HsIn r;
+  r.norm = gamma.has_value();
+  r.M = x.size(0), r.K = x.size(1);
+  MX_CHECK(w.is_cuda() && w.scalar_type() == at::kBFloat16 && w.dim() == 2 && w.stride(1) == 1 && w.size(1) == r.K &&
+               aligned16(w) && aligned16(x) && x.dim() == 2, "fused decode GEMM: x [M, K], w bf16 [N, K]");
+  if (!r.norm) {
+    MX_CHECK(x.is_cuda() && x.scalar_type() == at::kBFloat16 && x.stride(1) == 1 && !delta.has_value(), "x bf16 rows");
+    r.x = bf(x), r.ldx = x.stride(0);
+    return r;
+  }
+  check_f32(x, "h");
+  check_f32(*gamma, "gamma");
+  MX_CHECK(gamma->numel() == r.K, "gamma [K]");
+  r.h = x.data_ptr<float>(), r.gamma = gamma->data_ptr<float>();
+  r.hn = x;
+  if (delta.has_value()) {
+    MX_CHECK(delta->is_cuda() && delta->scalar_type() == at::kBFloat16 && delta->sizes() == x.sizes() &&
+                 delta->stride(1) == 1 && aligned16(*delta), "delta bf16 [M, K] rows");
+    r.delta = bf(*delta), r.ldd = delta->stride(0);
+    r.hn = at::empty_like(x);
+    r.h_out = r.hn.data_ptr<float>();
+  }
+  return r;
+}
+
+// (group_norm(h + delta) * gamma) . w^T and the new residual
+std::tuple<at::Tensor, at::Tensor> hs_norm_linear(const c10::optional<at::Tensor>& delta, const at::Tensor& h,
+                                                  const at::Tensor& gamma, int64_t groups, double eps,
+                                                  const at::Tensor& w) {
+  DevGuard g(w.device());
+  HsIn i = hs_in(h, delta, gamma, w);
+  auto y = at::empty({i.M, w.size(0)}, w.options());
+  MX_OK(mx_hs_norm_gemm(i.delta, i.ldd, i.h, i.gamma, i.h_out, (int)groups, (float)eps, bf(w), w.stride(0), bfm(y),
+                        w.size(0), (int)i.M, (int)w.size(0), (int)i.K, cur_stream()));
+  return {y, i.hn};
+}
+
+at::Tensor hs_poly_linear(const at::Tensor& z, const at::Tensor& coef, double eps, const at::Tensor& w) {
+  DevGuard g(w.device());
+  check_f32(coef, "coef");
+  MX_CHECK(coef.numel() == 4, "four coefficients");
+  HsIn i = hs_in(z, c10::nullopt, c10::nullopt, w);
+  auto y = at::empty({i.M, w.size(0)}, w.options());
+  MX_OK(mx_hs_poly_gemm(i.x, i.ldx, coef.data_ptr<float>(), (float)eps, bf(w), w.stride(0), bfm(y), w.size(0), (int)i.M,
+                        (int)w.size(0), (int)i.K, cur_stream()));
+  return y;
+}
+
+// x: bf16 rows, or with gamma the f32 residual; w [3 W, K]
+std::tuple<at::Tensor, at::Tensor> hs_gru_linear(const c10::optional<at::Tensor>& delta, const at::Tensor& x,
+                                                 const c10::optional<at::Tensor>& gamma, int64_t groups, double eps,
+                                                 const at::Tensor& w, const at::Tensor& bias, const at::Tensor& slots,
+                                                 at::Tensor state) {
+  DevGuard g(w.device());
+  HsIn i = hs_in(x, delta, gamma, w);
+  const int64_t W = w.size(0) / 3;
+  check_f32(bias, "bias");
+  check_f32(state, "state");
+  MX_CHECK(w.size(0) == 3 * W && bias.numel() == 2 * W && state.dim() == 2 && state.size(1) == W, "minGRU shapes");
+  auto y = at::empty({i.M, W}, w.options());
+  MX_OK(mx_hs_gru_gemm(i.x, i.ldx, i.norm, i.delta, i.ldd, i.h, i.gamma, i.h_out, (int)groups, (float)eps, bf(w),
+                       w.stride(0), bias.data_ptr<float>(), i32(slots, "slots", i.M), state.data_ptr<float>(), bfm(y),
+                       (int)i.M, (int)W, (int)i.K, cur_stream()));
+  return {y, i.norm ? i.hn : x};
+}
+
 mx::ConvRope conv_args(const at::Tensor& x, const at::Tensor& w, const at::Tensor& cos, const at::Tensor& sin,
                        int64_t rd, int64_t H, int64_t G, int64_t D, int64_t E) {
   act_f32(x, "x");
@@ -69,14 +146,14 @@ mx::ConvRope conv_args(const at::Tensor& x, const at::Tensor& w, const at::Tenso
   check_f32(cos, "cos");
   check_f32(sin, "sin");
   const int64_t C = (H + G) * D + G * E;
-  MX_CHECK(w.dim() == 2 && w.size(0) == C, "conv w [C, taps]");
+  MX_CHECK(w.dim() == 2 && w.size(1) == C, "conv w [taps, C]");
   MX_CHECK(cos.dim() == 2 && cos.size(1) == rd / 2 && sin.sizes() == cos.sizes(), "cos / sin [max_pos, rd / 2]");
   mx::ConvRope a = {};
   a.ldx = act_rows(x, "x");
   MX_CHECK(x.size(1) >= C && aligned16(x), "x [rows, >= C], 16-byte aligned");
   a.x = x.data_ptr();
   a.w = w.data_ptr<float>();
-  a.taps = (int)w.size(1);
+  a.taps = (int)w.size(0);
   a.cosb = cos.data_ptr<float>();
   a.sinb = sin.data_ptr<float>();
   a.rd = (int)rd, a.H = (int)H, a.G = (int)G, a.D = (int)D, a.E = (int)E;
@@ -100,8 +177,7 @@ void conv_cache(mx::ConvRope& a, const at::Tensor& x, at::Tensor& kc, at::Tensor
 // -> q [H, T, Dp], k [G, T, Dp], v [G, T, Ep], convolved and rotated; padding dims are zero
 std::tuple<at::Tensor, at::Tensor, at::Tensor> conv_rope_prefill(
     const at::Tensor& x, const at::Tensor& w, const at::Tensor& cos, const at::Tensor& sin, int64_t rd, int64_t H,
-    int64_t G, int64_t D, int64_t E, int64_t Dp, int64_t Ep, const at::Tensor& rowpos, const at::Tensor& rowseq,
-    const at::Tensor& seqs, int64_t chunk, const c10::optional<at::Tensor>& kc, const c10::optional<at::Tensor>& vc,
+    int64_t G, int64_t D, int64_t E, int64_t Dp, int64_t Ep, const at::Tensor& rows, int64_t chunk, const c10::optional<at::Tensor>& kc, const c10::optional<at::Tensor>& vc,
     const c10::optional<at::Tensor>& bt, const c10::optional<at::Tensor>& ring) {
   DevGuard g(x.device());
   mx::ConvRope a = conv_args(x, w, cos, sin, rd, H, G, D, E);
@@ -119,10 +195,7 @@ std::tuple<at::Tensor, at::Tensor, at::Tensor> conv_rope_prefill(
     conv_cache(a, x, kt, vt, *bt, rt);
     MX_CHECK(a.Dp == Dp && a.Ep == Ep, "cache rows as wide as the outputs");
   }
-  const int32_t* rp = i32(rowpos, "rowpos", T);
-  const int32_t* rs = i32(rowseq, "rowseq", T);
-  const int32_t* sq = i32(seqs, "seqs", 2);
-  MX_OK(mx_conv_rope_prefill(&a, x.scalar_type() == at::kFloat, rp, rs, sq, (int)T, cur_stream()));
+  MX_OK(mx_conv_rope_prefill(&a, x.scalar_type() == at::kFloat, i32(rows, "rows", 4 * T), (int)T, cur_stream()));
   return {q, k, v};
 }
 
@@ -141,6 +214,35 @@ at::Tensor conv_rope_decode(const at::Tensor& x, const at::Tensor& w, const at::
   MX_OK(mx_conv_rope_decode(&a, x.scalar_type() == at::kFloat, i32(pos, "pos", B), i32(slots, "slots", B), (int)B,
                             cur_stream()));
   return q;
+}
+
+// w [C + H E, K] (q | k | v | gate) -> (q [M, H, Dp], gate [M, H E], new residual)
+std::tuple<at::Tensor, at::Tensor, at::Tensor> hs_conv_linear(
+    const c10::optional<at::Tensor>& delta, const at::Tensor& x, const c10::optional<at::Tensor>& gamma,
+    int64_t groups, double eps, const at::Tensor& w, const at::Tensor& cw, const at::Tensor& cos, const at::Tensor& sin,
+    int64_t rd, int64_t H, int64_t G, int64_t D, int64_t E, const at::Tensor& pos, const at::Tensor& slots,
+    int64_t chunk, at::Tensor kc, at::Tensor vc, const at::Tensor& bt, at::Tensor ring) {
+  DevGuard g(w.device());
+  HsIn i = hs_in(x, delta, gamma, w);
+  mx::ConvRope a = {};
+  check_f32(cw, "conv w");
+  check_f32(cos, "cos");
+  check_f32(sin, "sin");
+  const int64_t C = (H + G) * D + G * E;
+  MX_CHECK(cw.dim() == 2 && cw.size(1) == C && w.size(0) == C + H * E, "conv w [taps, C], w [C + H E, K]");
+  MX_CHECK(cos.dim() == 2 && cos.size(1) == rd / 2 && sin.sizes() == cos.sizes(), "cos / sin [max_pos, rd / 2]");
+  MX_CHECK(chunk > 0 && chunk <= INT32_MAX, "chunk");
+  a.w = cw.data_ptr<float>(), a.taps = (int)cw.size(0);
+  a.cosb = cos.data_ptr<float>(), a.sinb = sin.data_ptr<float>();
+  a.rd = (int)rd, a.H = (int)H, a.G = (int)G, a.D = (int)D, a.E = (int)E, a.chunk = (int)chunk;
+  conv_cache(a, w, kc, vc, bt, ring);
+  auto q = at::empty({i.M, H, (int64_t)a.Dp}, w.options());
+  auto gate = at::empty({i.M, H * E}, w.options());
+  a.q = q.data_ptr(), a.qh = a.Dp, a.qt = H * a.Dp;
+  MX_OK(mx_hs_conv_gemm(i.x, i.ldx, i.norm, i.delta, i.ldd, i.h, i.gamma, i.h_out, (int)groups, (float)eps, bf(w),
+                        w.stride(0), &a, i32(pos, "pos", i.M), i32(slots, "slots", i.M), bfm(gate), (int)i.M, (int)i.K,
+                        cur_stream()));
+  return {q, gate, i.norm ? i.hn : x};
 }
 
 const void* gate_ptr(const at::Tensor& gate, const at::Tensor& like, int64_t rows, int64_t cols, int64_t& ld) {
@@ -281,13 +383,17 @@ at::Tensor poly_norm(const at::Tensor& z, const at::Tensor& coef, double eps) {
 TORCH_LIBRARY_FRAGMENT(mxllm, m) {
   m.def("embed_rows(Tensor ids, Tensor w) -> Tensor");
   m.def("group_norm(Tensor? delta, Tensor(a!) h, Tensor w, int groups, float eps, bool f32) -> Tensor");
-  m.def("conv_rope_prefill(Tensor x, Tensor w, Tensor cos, Tensor sin, int rd, int H, int G, int D, int E, int Dp, int Ep, Tensor rowpos, Tensor rowseq, Tensor seqs, int chunk, Tensor(a!)? kc=None, Tensor(b!)? vc=None, Tensor? bt=None, Tensor(c!)? ring=None) -> (Tensor, Tensor, Tensor)");
+  m.def("conv_rope_prefill(Tensor x, Tensor w, Tensor cos, Tensor sin, int rd, int H, int G, int D, int E, int Dp, int Ep, Tensor rows, int chunk, Tensor(a!)? kc=None, Tensor(b!)? vc=None, Tensor? bt=None, Tensor(c!)? ring=None) -> (Tensor, Tensor, Tensor)");
   m.def("conv_rope_decode(Tensor x, Tensor w, Tensor cos, Tensor sin, int rd, int H, int G, int D, int E, Tensor pos, Tensor slots, int chunk, Tensor(a!) kc, Tensor(b!) vc, Tensor bt, Tensor(c!) ring) -> Tensor");
   m.def("attn_seg(Tensor q, Tensor k, Tensor v, Tensor blocks, Tensor gate, int E, float scale) -> Tensor");
   m.def("chunk_attn(Tensor q, Tensor k, Tensor v, Tensor pos, Tensor gate, int D, int E, int chunk, float scale, Tensor? slots=None, Tensor? bt=None) -> Tensor");
   m.def("attn_combine(Tensor ml, Tensor po, Tensor gate, int E) -> Tensor");
   m.def("mingru_scan(Tensor x, Tensor bias, Tensor chunks, Tensor seqs, bool multi, Tensor(a!)? state=None) -> Tensor");
   m.def("mingru_step(Tensor x, Tensor bias, Tensor slots, Tensor(a!) state) -> Tensor");
+  m.def("hs_norm_linear(Tensor? delta, Tensor h, Tensor gamma, int groups, float eps, Tensor w) -> (Tensor, Tensor)");
+  m.def("hs_poly_linear(Tensor z, Tensor coef, float eps, Tensor w) -> Tensor");
+  m.def("hs_gru_linear(Tensor? delta, Tensor x, Tensor? gamma, int groups, float eps, Tensor w, Tensor bias, Tensor slots, Tensor(a!) state) -> (Tensor, Tensor)");
+  m.def("hs_conv_linear(Tensor? delta, Tensor x, Tensor? gamma, int groups, float eps, Tensor w, Tensor cw, Tensor cos, Tensor sin, int rd, int H, int G, int D, int E, Tensor pos, Tensor slots, int chunk, Tensor(a!) kc, Tensor(b!) vc, Tensor bt, Tensor(c!) ring) -> (Tensor, Tensor, Tensor)");
   m.def("poly_norm(Tensor z, Tensor coef, float eps) -> Tensor");
 }
 
@@ -301,5 +407,9 @@ TORCH_LIBRARY_IMPL(mxllm, CUDA, m) {
   m.impl("attn_combine", &attn_combine);
   m.impl("mingru_scan", &mingru_scan);
   m.impl("mingru_step", &mingru_step);
+  m.impl("hs_norm_linear", &hs_norm_linear);
+  m.impl("hs_poly_linear", &hs_poly_linear);
+  m.impl("hs_gru_linear", &hs_gru_linear);
+  m.impl("hs_conv_linear", &hs_conv_linear);
   m.impl("poly_norm", &poly_norm);
 }

@@ -8,7 +8,7 @@ namespace mx {
 struct ConvRope {
   const void* x;        // [rows, ldx]: q | k | v projections side by side
   int64_t ldx;
-  const float* w;       // [C, taps], C = (H + G) D + G E
+  const float* w;       // [taps, C], C = (H + G) D + G E
   int taps;
   const float* cosb;    // [max_pos, rd / 2]
   const float* sinb;

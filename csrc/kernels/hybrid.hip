@@ -120,19 +120,35 @@ __device__ __forceinline__ void stn(T* p, int n, const float (&v)[VEC]) {
   }
 }
 
-// rotate and store the convolved channels y of (row, position p, cache slot); keep: into the cache
+// rotate and store the convolved channels y of (row, position p); cr: the cache row (slot, head, p),
+// or -1 (not kept)
 template <int VEC, typename T>
 __device__ __forceinline__ void conv_finish(const ConvRope& a, int sec, int head, int d0, int n, int64_t row, int p,
-                                            int slot, bool keep, float (&y)[VEC]) {
-  if (sec < 2) {
+                                            int64_t cr, float (&y)[VEC]) {
+  if (sec < 2 && d0 < a.rd) {
+    const int64_t t = (int64_t)p * (a.rd >> 1) + (d0 >> 1);
+    if constexpr (VEC == 8) {
+      if ((a.rd & 7) == 0) {  // four whole pairs: 16-byte table reads
+        float c[4], s[4];
+        ldv<4>(a.cosb + t, c);
+        ldv<4>(a.sinb + t, s);
 #pragma unroll
-    for (int i = 0; i + 1 < VEC; i += 2) {
-      const int d = d0 + i;
-      if (d + 1 < a.rd) {
-        const float c = a.cosb[(int64_t)p * (a.rd >> 1) + (d >> 1)], s = a.sinb[(int64_t)p * (a.rd >> 1) + (d >> 1)];
-        const float u = y[i], v = y[i + 1];
-        y[i] = u * c - v * s;
-        y[i + 1] = v * c + u * s;
+        for (int i = 0; i < 4; ++i) {
+          const float u = y[2 * i], v = y[2 * i + 1];
+          y[2 * i] = u * c[i] - v * s[i];
+          y[2 * i + 1] = v * c[i] + u * s[i];
+        }
+      }
+    }
+    if (VEC != 8 || (a.rd & 7)) {
+#pragma unroll
+      for (int i = 0; i + 1 < VEC; i += 2) {
+        if (d0 + i + 1 < a.rd) {
+          const float c = a.cosb[t + (i >> 1)], s = a.sinb[t + (i >> 1)];
+          const float u = y[i], v = y[i + 1];
+          y[i] = u * c - v * s;
+          y[i + 1] = v * c + u * s;
+        }
       }
     }
   }
@@ -145,19 +161,21 @@ __device__ __forceinline__ void conv_finish(const ConvRope& a, int sec, int head
     if (d0 + VEC >= dim)  // the head's last channels: its padding too
       for (int d = dim; d < Wp; ++d) st1(out + d, 0.f);
   }
-  if (sec == 0) return;
-  T* cache = reinterpret_cast<T*>(sec == 1 ? a.kc : a.vc);
-  if (cache && keep)
-    stn<VEC>(cache + kv_row(a.bt, a.maxb, a.block, slot, a.G, head, p % a.chunk) * Wp + d0, n, y);
+  if (sec > 0 && cr >= 0) stn<VEC>(reinterpret_cast<T*>(sec == 1 ? a.kc : a.vc) + cr * Wp + d0, n, y);
 }
 
-// prompt rows: rowpos [T] position, rowseq [T] sequence, seqs [n, 2] = (slot or -1, length).
-// One thread walks RUN consecutive rows of VEC channels with the last taps - 1 rows in registers.
-constexpr int kConvRun = 8;
+// VEC consecutive channels of one tap's weights
+template <int VEC>
+__device__ __forceinline__ void conv_taps(const float* w, int n, float (&v)[VEC]) {
+  ldn<VEC>(w, n, v);
+}
+
+// prompt rows: rows [T] = (position, slot or -1, sequence length, -).  One thread walks RUN consecutive
+// rows of VEC channels with the last taps - 1 rows in registers.
+constexpr int kConvRun = 16;
 template <int VEC, typename T, int TAPS>
-__global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, const int32_t* __restrict__ rowpos,
-                                                                const int32_t* __restrict__ rowseq,
-                                                                const int32_t* __restrict__ seqs, int T_, int nvec) {
+__global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, const int4* __restrict__ rows, int T_,
+                                                                int nvec) {
   const int f = blockIdx.x * 256 + threadIdx.x;
   if (f >= nvec) return;
   int sec, head, d0, ch, dim;
@@ -167,12 +185,21 @@ __global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, cons
   const int C = (a.H + a.G) * a.D + a.G * a.E;
   const int taps = TAPS ? TAPS : a.taps;
   const int r0 = blockIdx.y * kConvRun, r1 = min(T_, r0 + kConvRun);
+  auto finish = [&](int r, const int4& ri, const float (&u)[VEC], float (&y)[VEC]) {
+    const int p = ri.x, slot = ri.y, S = ri.z;
+    int64_t cr = -1;
+    if (slot >= 0 && a.kc) {
+      if (p >= S - taps)
+        stn<VEC>(reinterpret_cast<T*>(a.ring) + ((int64_t)slot * taps + p % taps) * C + ch, n, u);
+      if (sec > 0 && p >= S / a.chunk * a.chunk)  // the chunk the next token belongs to
+        cr = kv_row(a.bt, a.maxb, a.block, slot, a.G, head, p % a.chunk);
+    }
+    conv_finish<VEC, T>(a, sec, head, d0, n, r, p, cr, y);
+  };
   if constexpr (TAPS > 0) {
     float wt[TAPS][VEC], win[TAPS][VEC];  // win[j]: row r - (TAPS - 1) + j
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j)
-#pragma unroll
-      for (int i = 0; i < VEC; ++i) wt[j][i] = i < n ? a.w[(int64_t)(ch + i) * TAPS + j] : 0.f;
+    for (int j = 0; j < TAPS; ++j) conv_taps<VEC>(a.w + (int64_t)j * C + ch, n, wt[j]);
 #pragma unroll
     for (int j = 1; j < TAPS; ++j) {
       const int r = r0 - TAPS + j;
@@ -181,43 +208,40 @@ __global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, cons
 #pragma unroll
         for (int i = 0; i < VEC; ++i) win[j][i] = 0.f;
     }
+#pragma unroll 4
     for (int r = r0; r < r1; ++r) {
 #pragma unroll
       for (int j = 0; j + 1 < TAPS; ++j)
 #pragma unroll
         for (int i = 0; i < VEC; ++i) win[j][i] = win[j + 1][i];
       ldn<VEC>(x + r * a.ldx, n, win[TAPS - 1]);
-      const int p = rowpos[r], sq = rowseq[r], slot = seqs[2 * sq], S = seqs[2 * sq + 1];
+      const int4 ri = rows[r];
       float y[VEC];
 #pragma unroll
       for (int i = 0; i < VEC; ++i) y[i] = 0.f;
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j)
-        if (p >= TAPS - 1 - j)  // the row TAPS - 1 - j back is of this sequence
+      for (int j = 0; j < TAPS; ++j) {
+        const float on = ri.x >= TAPS - 1 - j ? 1.f : 0.f;  // is the row TAPS - 1 - j back of this sequence?
 #pragma unroll
-          for (int i = 0; i < VEC; ++i) y[i] += wt[j][i] * win[j][i];
-      if (slot >= 0 && a.ring && p >= S - taps)
-        stn<VEC>(reinterpret_cast<T*>(a.ring) + ((int64_t)slot * taps + p % taps) * C + ch, n, win[TAPS - 1]);
-      conv_finish<VEC, T>(a, sec, head, d0, n, r, p, slot, slot >= 0 && p >= S / a.chunk * a.chunk, y);
+        for (int i = 0; i < VEC; ++i) y[i] += wt[j][i] * (on != 0.f ? win[j][i] : 0.f);
+      }
+      finish(r, ri, win[TAPS - 1], y);
     }
   } else {
     for (int r = r0; r < r1; ++r) {
-      const int p = rowpos[r], sq = rowseq[r], slot = seqs[2 * sq], S = seqs[2 * sq + 1];
-      float y[VEC], u[VEC];
+      const int4 ri = rows[r];
+      float y[VEC], u[VEC], wv[VEC];
 #pragma unroll
       for (int i = 0; i < VEC; ++i) y[i] = 0.f;
       for (int j = 0; j < taps; ++j) {
         const int back = taps - 1 - j;
-        if (p < back) continue;
+        if (ri.x < back) continue;
         ldn<VEC>(x + (int64_t)(r - back) * a.ldx, n, u);
+        conv_taps<VEC>(a.w + (int64_t)j * C + ch, n, wv);
 #pragma unroll
-        for (int i = 0; i < VEC; ++i) y[i] += (i < n ? a.w[(int64_t)(ch + i) * taps + j] : 0.f) * u[i];
+        for (int i = 0; i < VEC; ++i) y[i] += wv[i] * u[i];
       }
-      if (slot >= 0 && a.ring && p >= S - taps) {
-        ldn<VEC>(x + (int64_t)r * a.ldx, n, u);
-        stn<VEC>(reinterpret_cast<T*>(a.ring) + ((int64_t)slot * taps + p % taps) * C + ch, n, u);
-      }
-      conv_finish<VEC, T>(a, sec, head, d0, n, r, p, slot, slot >= 0 && p >= S / a.chunk * a.chunk, y);
+      finish(r, ri, u, y);  // u: the row itself (the last tap)
     }
   }
 }
@@ -235,31 +259,36 @@ __global__ void __launch_bounds__(64) conv_rope_decode_kernel(ConvRope a, const 
   T* ring = reinterpret_cast<T*>(a.ring) + (int64_t)slot * a.taps * C + ch;
   float u[VEC], y[VEC];
   ldn<VEC>(reinterpret_cast<const T*>(a.x) + (int64_t)b * a.ldx + ch, n, u);
+  float wv[VEC];
+  conv_taps<VEC>(a.w + (int64_t)(a.taps - 1) * C + ch, n, wv);
 #pragma unroll
-  for (int i = 0; i < VEC; ++i) y[i] = (i < n ? a.w[(int64_t)(ch + i) * a.taps + a.taps - 1] : 0.f) * u[i];
+  for (int i = 0; i < VEC; ++i) y[i] = wv[i] * u[i];
   for (int back = 1; back < a.taps && back <= p; ++back) {
     float o[VEC];
     ldn<VEC>(ring + (int64_t)((p - back) % a.taps) * C, n, o);
+    conv_taps<VEC>(a.w + (int64_t)(a.taps - 1 - back) * C + ch, n, wv);
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) y[i] += (i < n ? a.w[(int64_t)(ch + i) * a.taps + a.taps - 1 - back] : 0.f) * o[i];
+    for (int i = 0; i < VEC; ++i) y[i] += wv[i] * o[i];
   }
   stn<VEC>(ring + (int64_t)(p % a.taps) * C, n, u);
-  conv_finish<VEC, T>(a, sec, head, d0, n, b, p, slot, true, y);
+  conv_finish<VEC, T>(a, sec, head, d0, n, b, p,
+                      sec > 0 ? kv_row(a.bt, a.maxb, a.block, slot, a.G, head, p % a.chunk) : -1, y);
 }
 
 // ------------------------------------------------------------------ PolyNorm
-// y = a N(z) + b N(z^2) + c N(z^3) + e, N over the whole row; coef = (a, b, c, e)
-template <typename T, int VEC>
-__global__ void __launch_bounds__(256) poly_norm_kernel(const T* __restrict__ z, int64_t ldz,
-                                                        const float* __restrict__ coef, T* __restrict__ y, int F,
-                                                        float eps) {
-  __shared__ float scratch[16];
+// y = a N(z) + b N(z^2) + c N(z^3) + e, N over the whole row; coef = (a, b, c, e).  One workgroup of
+// NT threads per row; ITERS > 0: the row stays in registers (one read), 0: read twice.
+template <typename T, int VEC, int NT, int ITERS>
+__global__ void __launch_bounds__(NT) poly_norm_kernel(const T* __restrict__ z, int64_t ldz,
+                                                       const float* __restrict__ coef, T* __restrict__ y, int F,
+                                                       float eps) {
+  __shared__ float red[3][16];
+  constexpr int KEEP = ITERS > 0 ? ITERS : 1;
+  typedef T vt __attribute__((ext_vector_type(VEC > 1 ? VEC : 2)));
   const T* zp = z + (int64_t)blockIdx.x * ldz;
   T* yp = y + (int64_t)blockIdx.x * F;
   float s1 = 0.f, s2 = 0.f, s3 = 0.f;
-  for (int c = threadIdx.x * VEC; c < F; c += 256 * VEC) {
-    float v[VEC];
-    ldv<VEC>(zp + c, v);
+  auto add = [&](const float (&v)[VEC]) {
 #pragma unroll
     for (int i = 0; i < VEC; ++i) {
       const float q = v[i] * v[i];
@@ -267,19 +296,57 @@ __global__ void __launch_bounds__(256) poly_norm_kernel(const T* __restrict__ z,
       s2 += q * q;
       s3 += q * q * q;
     }
+  };
+  vt keep[KEEP];
+  if constexpr (ITERS > 0) {
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      const int c = (it * NT + threadIdx.x) * VEC;
+      if (c < F) keep[it] = *reinterpret_cast<const vt*>(zp + c);
+      else keep[it] = 0;
+    }
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      float v[VEC];
+      ldv<VEC>(reinterpret_cast<const T*>(&keep[it]), v);
+      add(v);
+    }
+  } else {
+    for (int c = threadIdx.x * VEC; c < F; c += NT * VEC) {
+      float v[VEC];
+      ldv<VEC>(zp + c, v);
+      add(v);
+    }
   }
-  s1 = block_sum(s1, scratch);
-  s2 = block_sum(s2, scratch);
-  s3 = block_sum(s3, scratch);
+  s1 = wave_sum(s1), s2 = wave_sum(s2), s3 = wave_sum(s3);
+  if ((threadIdx.x & 63) == 0) red[0][threadIdx.x >> 6] = s1, red[1][threadIdx.x >> 6] = s2, red[2][threadIdx.x >> 6] = s3;
+  __syncthreads();
+  s1 = s2 = s3 = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; ++w) s1 += red[0][w], s2 += red[1][w], s3 += red[2][w];
   const float inv = 1.f / (float)F;
   const float k1 = coef[0] / sqrtf(s1 * inv + eps), k2 = coef[1] / sqrtf(s2 * inv + eps),
               k3 = coef[2] / sqrtf(s3 * inv + eps), e = coef[3];
-  for (int c = threadIdx.x * VEC; c < F; c += 256 * VEC) {
-    float v[VEC], o[VEC];
-    ldv<VEC>(zp + c, v);
+  auto put = [&](int c, const float (&v)[VEC]) {
+    float o[VEC];
 #pragma unroll
     for (int i = 0; i < VEC; ++i) o[i] = ((k3 * v[i] + k2) * v[i] + k1) * v[i] + e;
     stv<VEC>(yp + c, o);
+  };
+  if constexpr (ITERS > 0) {
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      const int c = (it * NT + threadIdx.x) * VEC;
+      float v[VEC];
+      ldv<VEC>(reinterpret_cast<const T*>(&keep[it]), v);
+      if (c < F) put(c, v);
+    }
+  } else {
+    for (int c = threadIdx.x * VEC; c < F; c += NT * VEC) {
+      float v[VEC];
+      ldv<VEC>(zp + c, v);
+      put(c, v);
+    }
   }
 }
 
@@ -363,14 +430,13 @@ static bool conv_v8(const ConvRope& a) {
 }
 
 
-extern "C" int mx_conv_rope_prefill(const ConvRope* pa, int f32, const int32_t* rowpos, const int32_t* rowseq,
-                                    const int32_t* seqs, int T, hipStream_t stream) {
+extern "C" int mx_conv_rope_prefill(const ConvRope* pa, int f32, const int32_t* rows, int T, hipStream_t stream) {
   if (T <= 0) return 0;
   const ConvRope& a = *pa;
   if (conv_check(a)) return -1;
 #define CP(VV, TT, TP)                                                                             \
   conv_rope_prefill_kernel<VV, TT, TP><<<dim3((conv_nvec<VV>(a) + 255) / 256, (T + kConvRun - 1) / kConvRun), 256, \
-                                         0, stream>>>(a, rowpos, rowseq, seqs, T, conv_nvec<VV>(a))
+                                         0, stream>>>(a, (const int4*)rows, T, conv_nvec<VV>(a))
 #define CPT(VV, TT)                                                                                \
   if (a.taps == 4) CP(VV, TT, 4); else if (a.taps == 3) CP(VV, TT, 3); else if (a.taps == 2) CP(VV, TT, 2); \
   else CP(VV, TT, 0)
@@ -402,15 +468,23 @@ extern "C" int mx_poly_norm(const void* z, int64_t ldz, const float* coef, void*
   if (T <= 0) return 0;
   if (F <= 0) return -1;
   const unsigned g = (unsigned)T;
+#define PN(TT, VV, NT, IT) poly_norm_kernel<TT, VV, NT, IT><<<g, NT, 0, stream>>>((const TT*)z, ldz, coef, (TT*)y, F, eps)
   if (f32) {
-    if (F % 4 == 0 && ldz % 4 == 0)
-      poly_norm_kernel<float, 4><<<g, 256, 0, stream>>>((const float*)z, ldz, coef, (float*)y, F, eps);
-    else poly_norm_kernel<float, 1><<<g, 256, 0, stream>>>((const float*)z, ldz, coef, (float*)y, F, eps);
+    if (F % 4 == 0 && ldz % 4 == 0) PN(float, 4, 256, 0); else PN(float, 1, 256, 0);
+  } else if (F % 8 || ldz % 8) {
+    PN(uint16_t, 1, 256, 0);
+  } else if (T <= 64 && F > 4096) {  // decode rows: latency
+    if (F <= 16384) PN(uint16_t, 8, 1024, 2); else if (F <= 32768) PN(uint16_t, 8, 1024, 4); else PN(uint16_t, 8, 1024, 0);
+  } else if (F <= 4096) {
+    PN(uint16_t, 8, 256, 2);
+  } else if (F <= 16384) {
+    PN(uint16_t, 8, 512, 4);
+  } else if (F <= 32768) {
+    PN(uint16_t, 8, 512, 8);
   } else {
-    if (F % 8 == 0 && ldz % 8 == 0)
-      poly_norm_kernel<uint16_t, 8><<<g, 256, 0, stream>>>((const uint16_t*)z, ldz, coef, (uint16_t*)y, F, eps);
-    else poly_norm_kernel<uint16_t, 1><<<g, 256, 0, stream>>>((const uint16_t*)z, ldz, coef, (uint16_t*)y, F, eps);
+    PN(uint16_t, 8, 256, 0);
   }
+#undef PN
   return (int)hipGetLastError();
 }
 

@@ -12,12 +12,40 @@
 
 namespace mx {
 
+// Tokens [t0, t0 + U) of NP projections (each W apart) of VEC channels, as stored; rows past n - 1
+// repeat the last one (loaded, not used).
+template <typename T, int VEC, int NP>
+struct Batch {
+  static constexpr int U = sizeof(T) == 2 ? 8 : 4;
+  typedef T vt __attribute__((ext_vector_type(VEC > 1 ? VEC : 2)));
+  vt r[U][NP];
+  __device__ __forceinline__ void load(const T* p, int64_t ldx, int W, int t0, int n) {
+#pragma unroll
+    for (int j = 0; j < U; ++j) {
+      const T* q = p + (int64_t)min(t0 + j, n - 1) * ldx;
+#pragma unroll
+      for (int k = 0; k < NP; ++k) {
+        if constexpr (VEC > 1) r[j][k] = *reinterpret_cast<const vt*>(q + (int64_t)k * W);
+        else r[j][k].x = q[(int64_t)k * W];
+      }
+    }
+  }
+  __device__ __forceinline__ void get(int j, int k, float (&v)[VEC]) const {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const T e = r[j][k][i];
+      v[i] = ld1(&e);
+    }
+  }
+};
+
 // chunks [nc, 4] = (first row, rows, sequence, 1 for the sequence's last chunk)
 template <typename T, int VEC>
 __global__ void __launch_bounds__(64) mingru_reduce_kernel(const T* __restrict__ x, int64_t ldx,
                                                            const float* __restrict__ bias,
                                                            const int32_t* __restrict__ chunks, float* __restrict__ prod,
                                                            float* __restrict__ part, int W) {
+  typedef Batch<T, VEC, 2> B;
   const int c = (blockIdx.x * 64 + threadIdx.x) * VEC, ck = blockIdx.y;
   if (c >= W || chunks[4 * ck + 3]) return;
   const int r0 = chunks[4 * ck], n = chunks[4 * ck + 1];
@@ -27,47 +55,73 @@ __global__ void __launch_bounds__(64) mingru_reduce_kernel(const T* __restrict__
 #pragma unroll
   for (int i = 0; i < VEC; ++i) a[i] = 1.f, s[i] = 0.f;
   const T* p = x + (int64_t)r0 * ldx + c;
-#pragma unroll 4
-  for (int t = 0; t < n; ++t) {
-    float z[VEC], u[VEC];
-    ldv<VEC>(p + (int64_t)t * ldx, z);
-    ldv<VEC>(p + (int64_t)t * ldx + W, u);
+  auto work = [&](const B& q, int t0) {
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) {
-      float keep, add;
-      mingru_gate<T>(z[i] + bz[i], u[i] + bu[i], keep, add);
-      a[i] *= keep;
-      s[i] = keep * s[i] + add;
+    for (int j = 0; j < B::U; ++j) {
+      if (t0 + j >= n) break;
+      float z[VEC], u[VEC];
+      q.get(j, 0, z);
+      q.get(j, 1, u);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) {
+        float keep, add;
+        mingru_gate<T>(z[i] + bz[i], u[i] + bu[i], keep, add);
+        a[i] *= keep;
+        s[i] = keep * s[i] + add;
+      }
     }
+  };
+  B q0, q1;  // one batch in flight while the other is folded in
+  q0.load(p, ldx, W, 0, n);
+  for (int t = 0; t < n; t += 2 * B::U) {
+    if (t + B::U < n) q1.load(p, ldx, W, t + B::U, n);
+    work(q0, t);
+    if (t + 2 * B::U < n) q0.load(p, ldx, W, t + 2 * B::U, n);
+    if (t + B::U < n) work(q1, t + B::U);
   }
   stv<VEC>(prod + (int64_t)ck * W + c, a);
   stv<VEC>(part + (int64_t)ck * W + c, s);
 }
 
-// seqs [n, 3] = (slot, first chunk, chunks): part[chunk] <- the state ahead of the chunk
-__global__ void __launch_bounds__(64) mingru_carry_kernel(const int32_t* __restrict__ seqs,
-                                                          const float* __restrict__ prod, float* __restrict__ part,
-                                                          int W) {
-  const int c = blockIdx.x * 64 + threadIdx.x, sq = blockIdx.y;
-  if (c >= W) return;
+// seqs [n, 3] = (slot, first chunk, chunks): part[chunk] <- the state ahead of the chunk.  A workgroup
+// takes 16 channels; its 16 thread groups compose 8 chunks each and meet in LDS, 128 chunks at a time.
+__global__ void __launch_bounds__(256) mingru_carry_kernel(const int32_t* __restrict__ seqs,
+                                                           const float* __restrict__ prod, float* __restrict__ part,
+                                                           int W) {
+  __shared__ float sa[16][16], sb[16][16];
+  const int cl = threadIdx.x & 15, g = threadIdx.x >> 4, sq = blockIdx.y;
+  const int c = blockIdx.x * 16 + cl;
+  const bool on = c < W;
   const int c0 = seqs[3 * sq + 1], n = seqs[3 * sq + 2];
-  float s = 0.f;
-  for (int k = 0; k < n; k += 8) {
-    float a[8], b[8];
+  float carry = 0.f;
+  for (int k0 = 0; k0 < n; k0 += 128) {
+    float a[8], b[8], A = 1.f, B = 0.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const bool on = k + j < n - 1;  // the last chunk's reduction is not formed
-      const int64_t o = (int64_t)(c0 + (on ? k + j : 0)) * W + c;
-      a[j] = on ? prod[o] : 0.f;
-      b[j] = on ? part[o] : 0.f;
+      const int k = k0 + 8 * g + j;
+      const bool live = on && k < n - 1;  // the last chunk is not reduced
+      const int64_t o = (int64_t)(c0 + k) * W + c;
+      a[j] = live ? prod[o] : 1.f;
+      b[j] = live ? part[o] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) A *= a[j], B = a[j] * B + b[j];
+    sa[g][cl] = A;
+    sb[g][cl] = B;
+    __syncthreads();
+    float s = carry;
+    for (int k = 0; k < 16; ++k) {
+      const float nx = sa[k][cl] * carry + sb[k][cl];
+      carry = nx;
+      if (k + 1 == g) s = nx;
     }
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      if (k + j < n) {
-        part[(int64_t)(c0 + k + j) * W + c] = s;
-        s = a[j] * s + b[j];
-      }
+      const int k = k0 + 8 * g + j;
+      if (on && k < n) part[(int64_t)(c0 + k) * W + c] = s;
+      s = a[j] * s + b[j];
     }
+    __syncthreads();
   }
 }
 
@@ -78,10 +132,14 @@ __global__ void __launch_bounds__(64) mingru_replay_kernel(const T* __restrict__
                                                            const int32_t* __restrict__ seqs,
                                                            const float* __restrict__ part, float* __restrict__ state,
                                                            T* __restrict__ y, int W) {
+  typedef Batch<T, VEC, 3> B;
   const int c = (blockIdx.x * 64 + threadIdx.x) * VEC, ck = blockIdx.y;
   if (c >= W) return;
   const int r0 = chunks[4 * ck], n = chunks[4 * ck + 1], sq = chunks[4 * ck + 2];
   float bz[VEC], bu[VEC], s[VEC];
+  const T* p = x + (int64_t)r0 * ldx + c;
+  B q0, q1;
+  q0.load(p, ldx, W, 0, n);
   ldv<VEC>(bias + c, bz);
   ldv<VEC>(bias + W + c, bu);
   if (ck == seqs[3 * sq + 1]) {
@@ -90,22 +148,30 @@ __global__ void __launch_bounds__(64) mingru_replay_kernel(const T* __restrict__
   } else {
     ldv<VEC>(part + (int64_t)ck * W + c, s);
   }
-  const T* p = x + (int64_t)r0 * ldx + c;
   T* o = y + (int64_t)r0 * W + c;
-#pragma unroll 4
-  for (int t = 0; t < n; ++t) {
-    float z[VEC], u[VEC], g[VEC], out[VEC];
-    ldv<VEC>(p + (int64_t)t * ldx, z);
-    ldv<VEC>(p + (int64_t)t * ldx + W, u);
-    ldv<VEC>(p + (int64_t)t * ldx + 2 * W, g);
+  auto work = [&](const B& q, int t0) {
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) {
-      float keep, add;
-      mingru_gate<T>(z[i] + bz[i], u[i] + bu[i], keep, add);
-      s[i] = keep * s[i] + add;
-      out[i] = s[i] * (g[i] * sigmoid_t<T>(g[i]));
+    for (int j = 0; j < B::U; ++j) {
+      if (t0 + j >= n) break;
+      float z[VEC], u[VEC], g[VEC], out[VEC];
+      q.get(j, 0, z);
+      q.get(j, 1, u);
+      q.get(j, 2, g);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) {
+        float keep, add;
+        mingru_gate<T>(z[i] + bz[i], u[i] + bu[i], keep, add);
+        s[i] = keep * s[i] + add;
+        out[i] = s[i] * (g[i] * sigmoid_t<T>(g[i]));
+      }
+      stv<VEC>(o + (int64_t)(t0 + j) * W, out);
     }
-    stv<VEC>(o + (int64_t)t * W, out);
+  };
+  for (int t = 0; t < n; t += 2 * B::U) {
+    if (t + B::U < n) q1.load(p, ldx, W, t + B::U, n);
+    work(q0, t);
+    if (t + 2 * B::U < n) q0.load(p, ldx, W, t + 2 * B::U, n);
+    if (t + B::U < n) work(q1, t + B::U);
   }
   const int slot = seqs[3 * sq];
   if (chunks[4 * ck + 3] && slot >= 0) stv<VEC>(state + (int64_t)slot * W + c, s);
@@ -155,7 +221,7 @@ extern "C" int mx_mingru_scan(const void* x, int64_t ldx, int f32, const float* 
     const dim3 grid((W + 64 * VV - 1) / (64 * VV), nc);                                                         \
     if (multi) {                                                                                                \
       mingru_reduce_kernel<TT, VV><<<grid, 64, 0, stream>>>((const TT*)x, ldx, bias, chunks, prod, part, W);    \
-      mingru_carry_kernel<<<dim3((W + 63) / 64, nseq), 64, 0, stream>>>(seqs, prod, part, W);                   \
+      mingru_carry_kernel<<<dim3((W + 15) / 16, nseq), 256, 0, stream>>>(seqs, prod, part, W);                   \
     }                                                                                                           \
     mingru_replay_kernel<TT, VV>                                                                                \
         <<<grid, 64, 0, stream>>>((const TT*)x, ldx, bias, chunks, seqs, part, state, (TT*)y, W);               \

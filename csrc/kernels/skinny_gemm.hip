@@ -31,15 +31,9 @@
 
 #include "common.h"
 #include "decode_fuse.h"
+#include "skinny_core.h"
 
 namespace mx {
-
-typedef __bf16 bf16x8_sk __attribute__((ext_vector_type(8)));
-
-__device__ __forceinline__ f32x4 mfma16_sk(const u16x8& a, const u16x8& b, const f32x4& c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_sk, a), __builtin_bit_cast(bf16x8_sk, b),
-                                                 c, 0, 0, 0);
-}
 
 // MB: 16-token blocks (1 or 2); X rows >= M are clamped to M-1 and discarded.
 // NC: 16-channel groups per workgroup: each X fragment then feeds NC MFMAs, so X traffic per
@@ -55,7 +49,7 @@ __global__ void __launch_bounds__(512) skinny_gemm_kernel(const uint16_t* __rest
   static_assert(!NORM || (MB == 1 && NC == 1), "fused RMSNorm: <= 16 rows, one channel group");
   static_assert(!MERGE || (MB == 1 && NC == 1 && !NORM && !SWO && !ROPE), "fused split merge: plain GEMM rows");
   constexpr bool LDSX = NORM || MERGE;  // X rows built in LDS by the prologue
-  constexpr int NW = 8, UNR = NC == 1 ? 8 : 4;
+  constexpr int NW = kSkWaves, UNR = sk_unr(NC);
   __shared__ f32x4 red[NW][NC][MB][64];
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -75,17 +69,7 @@ __global__ void __launch_bounds__(512) skinny_gemm_kernel(const uint16_t* __rest
   // NORM: the first UNR chunks' weight loads go out before the prologue, so the weight stream's
   // latency overlaps the RMSNorm instead of following it
   u16x8 apre[UNR][NC][2];
-  if constexpr (LDSX) {
-    if (nit >= UNR) {
-#pragma unroll
-      for (int u = 0; u < UNR; ++u)
-#pragma unroll
-        for (int j = 0; j < NC; ++j) {
-          apre[u][j][0] = *reinterpret_cast<const u16x8*>(wrow[j] + u * 64);
-          apre[u][j][1] = *reinterpret_cast<const u16x8*>(wrow[j] + u * 64 + 8);
-        }
-    }
-  }
+  if constexpr (LDSX) sk_prefetch<NC>(wrow, nit, apre);
   if constexpr (LDSX) {
     extern __shared__ __attribute__((aligned(16))) uint16_t xs[];  // [M, K] normalised / merged rows
     if constexpr (NORM) {
@@ -103,59 +87,7 @@ __global__ void __launch_bounds__(512) skinny_gemm_kernel(const uint16_t* __rest
   }
 
   f32x4 acc[NC][MB];
-#pragma unroll
-  for (int j = 0; j < NC; ++j)
-#pragma unroll
-    for (int mb = 0; mb < MB; ++mb) acc[j][mb] = f32x4{0.f, 0.f, 0.f, 0.f};
-  auto load = [&](int k, u16x8 (&a)[NC][2], u16x8 (&b)[MB][2]) {
-#pragma unroll
-    for (int j = 0; j < NC; ++j) {
-      a[j][0] = *reinterpret_cast<const u16x8*>(wrow[j] + k);
-      a[j][1] = *reinterpret_cast<const u16x8*>(wrow[j] + k + 8);
-    }
-#pragma unroll
-    for (int mb = 0; mb < MB; ++mb) {
-      b[mb][0] = *reinterpret_cast<const u16x8*>(xr[mb] + k);
-      b[mb][1] = *reinterpret_cast<const u16x8*>(xr[mb] + k + 8);
-    }
-  };
-  auto step = [&](const u16x8 (&a)[NC][2], const u16x8 (&b)[MB][2]) {
-#pragma unroll
-    for (int j = 0; j < NC; ++j)
-#pragma unroll
-      for (int mb = 0; mb < MB; ++mb) {
-        acc[j][mb] = mfma16_sk(a[j][0], b[mb][0], acc[j][mb]);
-        acc[j][mb] = mfma16_sk(a[j][1], b[mb][1], acc[j][mb]);
-      }
-  };
-  int it = 0;
-  if constexpr (LDSX) {
-    if (nit >= UNR) {  // first block: weights prefetched above, X fragments from LDS
-      u16x8 b[UNR][MB][2];
-#pragma unroll
-      for (int u = 0; u < UNR; ++u)
-#pragma unroll
-        for (int mb = 0; mb < MB; ++mb) {
-          b[u][mb][0] = *reinterpret_cast<const u16x8*>(xr[mb] + u * 64);
-          b[u][mb][1] = *reinterpret_cast<const u16x8*>(xr[mb] + u * 64 + 8);
-        }
-#pragma unroll
-      for (int u = 0; u < UNR; ++u) step(apre[u], b[u]);
-      it = UNR;
-    }
-  }
-  for (; it + UNR <= nit; it += UNR) {
-    u16x8 a[UNR][NC][2], b[UNR][MB][2];
-#pragma unroll
-    for (int u = 0; u < UNR; ++u) load((it + u) * 64, a[u], b[u]);
-#pragma unroll
-    for (int u = 0; u < UNR; ++u) step(a[u], b[u]);
-  }
-  for (; it < nit; ++it) {
-    u16x8 a[NC][2], b[MB][2];
-    load(it * 64, a, b);
-    step(a, b);
-  }
+  sk_stream<MB, NC, LDSX>(wrow, xr, nit, apre, acc);
   // C[row = channel 4g + i][col = token c] per (group, m-block): sum the NW K parts
 #pragma unroll
   for (int j = 0; j < NC; ++j)

@@ -110,7 +110,8 @@ class RevesunConfig:
 
 
 class RevesunLayer(nn.Module):
-    """``wx``: the projections of the normed input (z | u | gate, or q | k | v | gate); ``wo``: the
+    """``conv`` is kept as the checkpoint has it; the kernels read it tap by tap (``conv_t``).
+    ``wx``: the projections of the normed input (z | u | gate, or q | k | v | gate); ``wo``: the
     mixer's output; ``wup`` / ``wdown``: the feed-forward."""
 
     def __init__(self, spec: LayerSpec, h: int, *, dtype, device):
@@ -136,6 +137,14 @@ class RevesunLayer(nn.Module):
             self.wup = FusedLinear(h, [spec.ff], **kw)
             self.act = f32(4)
             self.wdown = FusedLinear(spec.ff, [h], **kw)
+
+
+    def conv_t(self) -> torch.Tensor:
+        """Convolution taps [taps, channels], rebuilt after the parameter was written."""
+        v = self.conv._version
+        if getattr(self, "_conv_t", None) is None or self._conv_t[0] != v or self._conv_t[1].device != self.conv.device:
+            self._conv_t = (v, self.conv.detach().t().contiguous())
+        return self._conv_t[1]
 
 
 class Revesun(nn.Module):
@@ -198,33 +207,59 @@ class Revesun(nn.Module):
         return have
 
     def prepare(self, max_seq: int) -> None:
-        """Size the rotation tables once (their storage must not move under a captured graph)."""
-        for s in self.cfg.layers:
+        """Build the derived tables once (their storage must not move under a captured graph)."""
+        for s, layer in zip(self.cfg.layers, self.layers):
             if s.kind == "attention":
                 self.rope(s, max_seq)
+                layer.conv_t()
 
     # ------------------------------------------------------------------ the layer stack
-    def _norm_proj(self, delta, h, gamma, lin) -> torch.Tensor:
-        return lin(hops.group_norm(delta, h, gamma, self.cfg.norm_groups, self.cfg.norm_eps, self.dtype))
+    def _norm_proj(self, delta, h, gamma, lin, fused: bool = False):
+        """(lin(norm(h + delta)), h + delta)."""
+        c = self.cfg
+        if fused:
+            r = hops.norm_linear(delta, h, gamma, c.norm_groups, c.norm_eps, plain_weight(lin))
+            if r is not None:
+                return r
+        return lin(hops.group_norm(delta, h, gamma, c.norm_groups, c.norm_eps, self.dtype)), h
+
+    def _mixer(self, i: int, delta, h, rows, n: int):
+        """(mixer output ahead of its output projection, h + delta)."""
+        layer, j, c = self.layers[i], self.kind_index[i], self.cfg
+        s = layer.spec
+        args = (delta, h, layer.norm1, c.norm_groups, c.norm_eps, plain_weight(layer.wx))
+        if s.kind == "mingru":
+            r = hops.gru_linear(*args, layer.bias, rows, j) if rows.decode else None
+            if r is not None:
+                return r
+            x, h = self._norm_proj(delta, h, layer.norm1, layer.wx)
+            return hops.min_gru(x, layer.bias, rows, j), h
+        cos, sin = self.rope(s, n)
+        r = hops.conv_linear(*args, layer.conv_t(), cos, sin, s.attn, rows, j) if rows.decode else None
+        if r is not None:
+            return r
+        x, h = self._norm_proj(delta, h, layer.norm1, layer.wx)
+        return hops.sink_attention(x, layer.conv_t(), cos, sin, s.attn, rows, j), h
+
+    def _down(self, z, layer, fused: bool):
+        if fused:
+            r = hops.poly_linear(z, layer.act, self.cfg.norm_eps, plain_weight(layer.wdown))
+            if r is not None:
+                return r
+        return layer.wdown(hops.poly_norm(z, layer.act, self.cfg.norm_eps))
 
     def rows(self, ids: torch.Tensor, rows, tap=None) -> torch.Tensor:
         """Final normed hidden rows of token ``ids`` [T] laid out as ``rows``.  ``tap(i, h)``: the
         residual stream after layer i (diagnostics)."""
         n = 0 if rows.decode else max(rows.lens)  # decode: the tables prepare() sized
         h = hops.embed_rows(ids, self.tok_emb)
-        delta = None
+        delta = None  # sub-block output not yet added to h
         for i, layer in enumerate(self.layers):
-            s, j = layer.spec, self.kind_index[i]
-            x = self._norm_proj(delta, h, layer.norm1, layer.wx)
-            if s.kind == "mingru":
-                y = hops.min_gru(x, layer.bias, rows, j)
-            else:
-                cos, sin = self.rope(s, n)
-                y = hops.sink_attention(x, layer.conv, cos, sin, s.attn, rows, j)
+            y, h = self._mixer(i, delta, h, rows, n)
             delta = layer.wo(y)
-            if s.ff:
-                z = self._norm_proj(delta, h, layer.norm2, layer.wup)
-                delta = layer.wdown(hops.poly_norm(z, layer.act, self.cfg.norm_eps))
+            if layer.spec.ff:
+                z, h = self._norm_proj(delta, h, layer.norm2, layer.wup, rows.decode)
+                delta = self._down(z, layer, rows.decode)
             if tap is not None:
                 tap(i, h + delta.float())
         return hops.group_norm(delta, h, self.final_norm, self.cfg.norm_groups, self.cfg.norm_eps, self.dtype)
@@ -242,6 +277,11 @@ class Revesun(nn.Module):
 
     def num_params(self, trainable_only: bool = False) -> int:
         return 0 if trainable_only else sum(p.numel() for p in self.parameters())
+
+
+def plain_weight(lin) -> torch.Tensor | None:
+    """The weight of an unquantised projection (what the fused decode kernels take)."""
+    return lin.weight if type(lin) is FusedLinear else None
 
 
 # ------------------------------------------------------------------ checkpoints

@@ -12,12 +12,14 @@ CPU tensors: plain PyTorch (the CPU test suite).
 """
 from __future__ import annotations
 
+import os
 from dataclasses import dataclass
 
 import numpy as np
 import torch
 
 from ._ext import native, use_native
+from .linear import NORM_M, SKINNY_M, _SKINNY_SMALL_W
 
 MFMA_MAX_DIM = 128  # widest head of the MFMA attention kernels
 MFMA_MAX_REP = 16   # query heads per key head in the split-K decode kernels
@@ -90,10 +92,12 @@ class PromptRows:
         self.offs = np.concatenate([[0], np.cumsum(self.lens)]).astype(np.int64)
         self.T = int(self.offs[-1])
         self._tables: dict = {}
-        pos = np.concatenate([np.arange(n, dtype=np.int32) for n in self.lens])
-        seq = np.repeat(np.arange(len(self.lens), dtype=np.int32), self.lens)
-        self.rowpos, self.rowseq = self._up(pos), self._up(seq)
-        self.seqs = self._up(np.array([self.slots, self.lens], dtype=np.int32).T)
+        # every row's (position, slot, sequence length, -)
+        info = np.zeros((self.T, 4), dtype=np.int32)
+        info[:, 0] = np.concatenate([np.arange(n) for n in self.lens])
+        info[:, 1] = np.repeat(self.slots, self.lens)
+        info[:, 2] = np.repeat(self.lens, self.lens)
+        self.rowinfo = self._up(info)
 
     def _up(self, a: np.ndarray) -> torch.Tensor:
         return torch.from_numpy(np.ascontiguousarray(a)).to(self.device)
@@ -212,7 +216,7 @@ def sink_attention(x: torch.Tensor, conv: torch.Tensor, cos: torch.Tensor, sin: 
                    layer: int) -> torch.Tensor:
     """x [T, q | k | v | gate] projections -> gated attention output [T, heads * vdim]: causal
     convolution of q, k, v over time, rotation of q and k, attention inside chunks with one added to
-    the softmax's denominator, times sigmoid(gate).  ``conv`` f32 [channels, taps]."""
+    the softmax's denominator, times sigmoid(gate).  ``conv`` f32 [taps, channels]."""
     C = sh.conv_channels
     gate = x[:, C:]
     H, G, D, E = sh.heads, sh.kv_heads, sh.dim, sh.vdim
@@ -224,10 +228,10 @@ def sink_attention(x: torch.Tensor, conv: torch.Tensor, cos: torch.Tensor, sin: 
     args = (x, conv, cos, sin, sh.rot_dims, H, G, D, E)
     if not rows.decode:
         keep = (c.k[layer], c.v[layer], c.bt, c.conv[layer]) if c is not None else ()
-        q, k, v = ops.conv_rope_prefill(*args, Dp, Ep, rows.rowpos, rows.rowseq, rows.seqs, sh.chunk, *keep)
+        q, k, v = ops.conv_rope_prefill(*args, Dp, Ep, rows.rowinfo, sh.chunk, *keep)
         if sh.mfma(x.dtype):
             return ops.attn_seg(q, k, v, rows.attn_blocks(sh.chunk), gate, E, sh.scale)
-        return ops.chunk_attn(q, k, v, rows.rowpos, gate, D, E, sh.chunk, sh.scale)
+        return ops.chunk_attn(q, k, v, rows.rowinfo[:, 0].contiguous(), gate, D, E, sh.chunk, sh.scale)
     q = ops.conv_rope_decode(*args, rows.pos, rows.slots, sh.chunk, c.k[layer], c.v[layer], c.bt, c.conv[layer])
     return decode_sink_attention(q, gate, sh, rows, layer)
 
@@ -242,6 +246,69 @@ def decode_sink_attention(q: torch.Tensor, gate: torch.Tensor, sh: AttnShape, ro
         return ops.attn_combine(ml, po, gate, sh.vdim)
     return ops.chunk_attn(q, c.k[layer], c.v[layer], rows.pos, gate, sh.dim, sh.vdim, sh.chunk, sh.scale, rows.slots,
                           c.bt)
+
+
+# ------------------------------------------------------------------ fused decode steps
+# csrc/kernels/hybrid_skinny.hip: the projections of up to SKINNY_M decode rows with the work after them
+# in the GEMM's epilogue, and for up to NORM_M rows the norm or activation ahead of them in its
+# prologue.  Each returns None where the kernel does not take the call (the caller runs the parts).
+# MXLLM_HYBRID_FUSED=0: always the parts (A/B).
+FUSED = os.environ.get("MXLLM_HYBRID_FUSED", "1") != "0"
+_NORM_MAX, _POLY_MAX = 16384, 32768  # rows x width held in LDS by a prologue
+
+
+def _fusable(t: torch.Tensor, w: torch.Tensor | None, mult: int = 16) -> bool:
+    M, K = t.shape
+    return bool(FUSED and w is not None and use_native(t) and w.dtype == torch.bfloat16 and 0 < M <= min(SKINNY_M, 16)
+                and K % 512 == 0 and w.shape[0] % mult == 0 and w.stride(1) == 1 and w.stride(0) % 8 == 0
+                and (M == 1 or w.numel() <= _SKINNY_SMALL_W))
+
+
+def _norm_fits(h: torch.Tensor, groups: int) -> bool:
+    M, K = h.shape
+    return M <= NORM_M and M * K <= _NORM_MAX and (K // groups) % 8 == 0 and M * groups <= 512
+
+
+def norm_linear(delta, h, gamma, groups: int, eps: float, w):
+    """(group_norm(h + delta) w^T, h + delta) in one launch."""
+    if not (_fusable(h, w) and _norm_fits(h, groups)):
+        return None
+    return native().hs_norm_linear(delta, h, gamma, groups, eps, w)
+
+
+def poly_linear(z, coef, eps: float, w):
+    """poly_norm(z) w^T in one launch."""
+    if not (_fusable(z, w) and z.shape[0] <= NORM_M and z.numel() <= _POLY_MAX):
+        return None
+    return native().hs_poly_linear(z, coef, eps, w)
+
+
+def _normed(delta, h, gamma, groups, eps):
+    """(delta, x, gamma) of a fused projection: the norm in its prologue, or run ahead of it."""
+    if _norm_fits(h, groups):
+        return delta, h, gamma
+    return None, group_norm(delta, h, gamma, groups, eps, torch.bfloat16), None
+
+
+def gru_linear(delta, h, gamma, groups: int, eps: float, w, bias, rows, layer: int):
+    """Decode: (minGRU output of the normed rows, new residual), state advanced; w = [z; u; gate]."""
+    if not (rows.decode and _fusable(h, w, 12)):
+        return None
+    d, x, g = _normed(delta, h, gamma, groups, eps)
+    y, hn = native().hs_gru_linear(d, x, g, groups, eps, w, bias, rows.slots, rows.caches.rec[layer])
+    return y, (hn if g is not None else h)
+
+
+def conv_linear(delta, h, gamma, groups: int, eps: float, w, conv, cos, sin, sh: AttnShape, rows, layer: int):
+    """Decode: (gated attention output of the normed rows, new residual); w = [q; k; v; gate]."""
+    if not (rows.decode and _fusable(h, w) and sh.dim % 4 == 0 and sh.vdim % 4 == 0):
+        return None
+    d, x, g = _normed(delta, h, gamma, groups, eps)
+    c = rows.caches
+    q, gate, hn = native().hs_conv_linear(d, x, g, groups, eps, w, conv, cos, sin, sh.rot_dims, sh.heads, sh.kv_heads,
+                                          sh.dim, sh.vdim, rows.pos, rows.slots, sh.chunk, c.k[layer], c.v[layer],
+                                          c.bt, c.conv[layer])
+    return decode_sink_attention(q, gate, sh, rows, layer), (hn if g is not None else h)
 
 
 # ------------------------------------------------------------------ CPU attention
@@ -271,9 +338,9 @@ def _sink_attention_ref(x, conv, cos, sin, sh: AttnShape, rows, layer: int) -> t
         return torch.matmul(w[:, None], vs.transpose(0, 1))[:, 0].reshape(-1)
 
     def token(u, hist, p):  # newest value u [C], hist: earlier ones newest first
-        y = conv[:, n - 1] * u
+        y = conv[n - 1] * u
         for back, o in enumerate(hist[:n - 1], 1):
-            y = y + conv[:, n - 1 - back] * o
+            y = y + conv[n - 1 - back] * o
         return (rot(y[:H * D].view(H, D), p).to(x.dtype).float(), rot(y[H * D:(H + G) * D].view(G, D), p),
                 y[(H + G) * D:].view(G, E))
 
