@@ -120,6 +120,25 @@ __device__ __forceinline__ void stn(T* p, int n, const float (&v)[VEC]) {
   }
 }
 
+// VEC channels of a row kept as stored (half the registers for bf16)
+template <typename T, int VEC>
+struct alignas(sizeof(T) * VEC) Piece {
+  T e[VEC];
+  __device__ __forceinline__ void load(const T* p, int n) {
+    if constexpr (VEC >= 4) {
+      typedef T vt __attribute__((ext_vector_type(VEC)));
+      *reinterpret_cast<vt*>(e) = *reinterpret_cast<const vt*>(p);
+    } else {
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) e[i] = i < n ? p[i] : T(0);
+    }
+  }
+  __device__ __forceinline__ void get(float (&v)[VEC]) const {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = ld1(e + i);
+  }
+};
+
 // rotate and store the convolved channels y of (row, position p); cr: the cache row (slot, head, p),
 // or -1 (not kept)
 template <int VEC, typename T>
@@ -172,7 +191,7 @@ __device__ __forceinline__ void conv_taps(const float* w, int n, float (&v)[VEC]
 
 // prompt rows: rows [T] = (position, slot or -1, sequence length, -).  One thread walks RUN consecutive
 // rows of VEC channels with the last taps - 1 rows in registers.
-constexpr int kConvRun = 16;
+constexpr int kConvRun = 8;
 template <int VEC, typename T, int TAPS>
 __global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, const int4* __restrict__ rows, int T_,
                                                                 int nvec) {
@@ -197,35 +216,29 @@ __global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, cons
     conv_finish<VEC, T>(a, sec, head, d0, n, r, p, cr, y);
   };
   if constexpr (TAPS > 0) {
-    float wt[TAPS][VEC], win[TAPS][VEC];  // win[j]: row r - (TAPS - 1) + j
+    float wt[TAPS][VEC];
+    Piece<T, VEC> win[TAPS - 1 + kConvRun];  // every row of the run and the ones ahead of it, in flight at once
+#pragma unroll
+    for (int j = 0; j < TAPS - 1 + kConvRun; ++j)
+      win[j].load(x + min(max(r0 - (TAPS - 1) + j, 0), T_ - 1) * a.ldx, n);  // rows outside: not used
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) conv_taps<VEC>(a.w + (int64_t)j * C + ch, n, wt[j]);
 #pragma unroll
-    for (int j = 1; j < TAPS; ++j) {
-      const int r = r0 - TAPS + j;
-      if (r >= 0) ldn<VEC>(x + r * a.ldx, n, win[j]);
-      else
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) win[j][i] = 0.f;
-    }
-#pragma unroll 4
-    for (int r = r0; r < r1; ++r) {
-#pragma unroll
-      for (int j = 0; j + 1 < TAPS; ++j)
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) win[j][i] = win[j + 1][i];
-      ldn<VEC>(x + r * a.ldx, n, win[TAPS - 1]);
+    for (int k = 0; k < kConvRun; ++k) {
+      const int r = r0 + k;
+      if (r >= r1) break;
       const int4 ri = rows[r];
-      float y[VEC];
+      float u[VEC], y[VEC];
 #pragma unroll
       for (int i = 0; i < VEC; ++i) y[i] = 0.f;
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
-        const float on = ri.x >= TAPS - 1 - j ? 1.f : 0.f;  // is the row TAPS - 1 - j back of this sequence?
+        if (ri.x < TAPS - 1 - j) continue;  // uniform: the row TAPS - 1 - j back is of an earlier sequence
+        win[k + j].get(u);
 #pragma unroll
-        for (int i = 0; i < VEC; ++i) y[i] += wt[j][i] * (on != 0.f ? win[j][i] : 0.f);
+        for (int i = 0; i < VEC; ++i) y[i] += wt[j][i] * u[i];
       }
-      finish(r, ri, win[TAPS - 1], y);
+      finish(r, ri, u, y);  // u: the row itself (the last tap)
     }
   } else {
     for (int r = r0; r < r1; ++r) {
