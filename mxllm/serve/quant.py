@@ -81,7 +81,7 @@ class W8Linear(nn.Module):
         M = x2.shape[0]
         if not use_native(x2):
             y = torch.matmul(x2, dequantize_e4m3(self.q, self.scale).to(x2.dtype).t())
-        elif M <= SMALL_M or self.in_features % 16:
+        elif M <= SMALL_M or self.in_features % 16 or self.out_features % 16:
             # weight-streaming HIP kernel: bf16 activations, weights dequantised in registers
             # (it falls back to dequantise + hipBLASLt for shapes it does not take)
             y = native().w8_linear(x2, self.q, self.scale)

@@ -119,3 +119,84 @@ def forward(cfg, weights, tokens, dt=torch.float64, collect=None):
         if collect is not None:
             collect.append(x.clone())
     return group_norm(x, w["final.norm"], groups, eps) @ w["embed"].T
+
+
+# ------------------------------------------------------------------ configurations and weights
+def attention(heads, kv, dim, vdim, conv, chunk, base, rdims, scale, ff=0):
+    return {"type": "attention", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv, "scale": scale,
+                      "mask": {"size": chunk}, "rot": {"base": base, "dims": rdims}}}
+
+
+def mingru(width, ff=0):
+    return {"type": "mingru", "mlp": {"kind": "dense", "ff": ff} if ff else None, "mixer": {"width": width}}
+
+
+def config(width, vocab, groups, layers, eps=1e-5):
+    return {"architecture": "Revesun", "width": width, "vocab": vocab, "norm": {"groups": groups, "eps": eps},
+            "layers": layers}
+
+
+def tensor_shapes(cfg):
+    h = cfg["width"]
+    out = {"embed": (cfg["vocab"], h), "final.norm": (h,)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", layer["mixer"]
+        out[p + "norm1"] = (h,)
+        if layer["type"] == "mingru":
+            w = mx["width"]
+            out.update({p + "mix.z": (w, h), p + "mix.z.b": (w,), p + "mix.x": (w, h), p + "mix.x.b": (w,),
+                        p + "mix.g": (w, h), p + "mix.o": (h, w)})
+        else:
+            rows = {"q": mx["heads"] * mx["dim"], "k": mx["kv_heads"] * mx["dim"], "v": mx["kv_heads"] * mx["vdim"]}
+            for n, r in rows.items():
+                out[p + f"mix.{n}"] = (r, h)
+                out[p + f"mix.{n}.conv"] = (r, mx["conv"])
+            out[p + "mix.g"] = (mx["heads"] * mx["vdim"], h)
+            out[p + "mix.o"] = (h, mx["heads"] * mx["vdim"])
+        if layer["mlp"]:
+            ff = layer["mlp"]["ff"]
+            out.update({p + "norm2": (h,), p + "mlp.up": (ff, h), p + "mlp.down": (h, ff), p + "mlp.act": (4,)})
+    return out
+
+
+def random_weights(cfg, seed=0):
+    """bf16 tensors under the checkpoint's names, scaled so that every term of a layer counts."""
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in tensor_shapes(cfg).items():
+        t = torch.randn(shape, generator=g)
+        if "norm" in name:
+            t = 1 + 0.2 * t
+        elif name.endswith(".conv"):
+            t = 0.3 * t
+            t[:, -1] += 1.0
+        elif name.endswith(".act"):
+            t = torch.tensor([0.6, 0.35, 0.25, 0.1]) + 0.05 * t
+        elif name.endswith(".b"):
+            t = 0.5 * t
+        elif len(shape) == 2:
+            t = t * (1.0 if name == "embed" else 1.3 / math.sqrt(shape[1]))
+        out[name] = t.to(torch.bfloat16)
+    return out
+
+
+def save(cfg, weights, path):
+    """Write a model directory."""
+    import json
+    import os
+
+    from safetensors.torch import save_file
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file(weights, os.path.join(path, "model.safetensors"))
+    return str(path)
+
+
+def greedy(cfg, weights, prompt, n, dt=torch.float64):
+    seq = list(prompt)
+    for _ in range(n):
+        seq.append(int(forward(cfg, weights, seq, dt)[-1].argmax()))
+    return seq[len(prompt):]
