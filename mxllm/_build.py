@@ -10,7 +10,11 @@ The HIP runtime is taken from torch's own ``torch/lib/libamdhip64.so``
 (same SONAME ``libamdhip64.so.7`` as /opt/rocm's), so the extension and torch
 share one runtime instance in-process.
 
-Usage: ``python -m mxllm._build [--force] [-j N]``.
+``COMPONENTS`` names subsets that also build on their own, into a library with the same op names:
+``serve`` has what a serving-only model needs, so a fresh checkout that only replays such a model
+(bin/trace_run) compiles a third of the sources.
+
+Usage: ``python -m mxllm._build [--force] [-j N] [--component serve]``.
 """
 from __future__ import annotations
 
@@ -28,6 +32,12 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 CSRC = os.path.join(ROOT, "csrc")
 OUT_DIR = os.path.join(ROOT, "build", "obj")
 LIB_PATH = os.path.join(ROOT, "mxllm", "_C.so")
+# component -> (library, kernel files, op binding files)
+COMPONENTS = {
+    "serve": (os.path.join(ROOT, "mxllm", "_C_serve.so"),
+              ("attn_fwd", "chunk_attn", "decode", "hybrid", "hybrid_skinny", "mingru", "sampling", "skinny_gemm"),
+              ("bindings_hybrid", "bindings_serve")),
+}
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 ARCH = os.environ.get("MXLLM_ARCH", "gfx950")
 
@@ -130,12 +140,18 @@ def _compile_checked(src: str, obj: str, cmd: list[str], flags: list[str]) -> st
     return _run([os.path.join(ROCM, "bin", "hipcc")] + flags + [fallback, "-c", src, "-o", obj])
 
 
-def build(force: bool = False, jobs: int = 8, verbose: bool = False) -> str:
+def build(force: bool = False, jobs: int = 8, verbose: bool = False, component: str | None = None) -> str:
+    """The whole library (``mxllm/_C.so``), or one of ``COMPONENTS``."""
     inc, tlib, abi = _torch_paths()
     os.makedirs(OUT_DIR, exist_ok=True)
     hdrs = sorted(glob.glob(os.path.join(CSRC, "**", "*.h"), recursive=True))
     hip_srcs = sorted(glob.glob(os.path.join(CSRC, "kernels", "*.hip")))
     cpp_srcs = sorted(glob.glob(os.path.join(CSRC, "*.cpp")) + glob.glob(os.path.join(CSRC, "runtime", "*.cpp")))
+    lib_path = LIB_PATH
+    if component is not None:
+        lib_path, kernels, cpps = COMPONENTS[component]
+        hip_srcs = [os.path.join(CSRC, "kernels", k + ".hip") for k in kernels]
+        cpp_srcs = [os.path.join(CSRC, c + ".cpp") for c in cpps]
     py_inc = sysconfig.get_paths()["include"]
 
     hip_flags = [
@@ -178,20 +194,22 @@ def build(force: bool = False, jobs: int = 8, verbose: bool = False) -> str:
                             print("[mxllm build] " + line[1:].replace("]", ":", 1), flush=True)
     objs = [j[1] for j in jobs_list]
     link_key = _hash([], "|".join(objs))
-    stamp = LIB_PATH + ".stamp"
-    if force or not os.path.exists(LIB_PATH) or not os.path.exists(stamp) or open(stamp).read() != link_key:
-        tmp = LIB_PATH + ".tmp"
+    stamp = lib_path + ".stamp"
+    if force or not os.path.exists(lib_path) or not os.path.exists(stamp) or open(stamp).read() != link_key:
+        tmp = f"{lib_path}.{os.getpid()}.tmp"
         cmd = (["g++", "-shared", "-o", tmp] + objs + [
             f"-L{tlib}", "-lc10", "-lc10_hip", "-ltorch", "-ltorch_cpu", "-ltorch_hip",
             f"{tlib}/libamdhip64.so", f"-Wl,-rpath,{tlib}", "-Wl,--no-as-needed",
         ])
         _run(cmd)
         _check_loadable(tmp)
-        os.replace(tmp, LIB_PATH)
+        os.replace(tmp, lib_path)
         with open(stamp, "w") as f:
             f.write(link_key)
         if verbose:
-            print(f"[mxllm build] linked {os.path.relpath(LIB_PATH, ROOT)}", flush=True)
+            print(f"[mxllm build] linked {os.path.relpath(lib_path, ROOT)}", flush=True)
+    if component is not None:
+        return lib_path
     _write_buildinfo(hip_srcs + cpp_srcs, hdrs, hip_flags, cxx_flags, len(todo), link_key)
     # drop stale objects from older source versions
     keep = set(objs)
@@ -236,8 +254,9 @@ def main(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--force", action="store_true")
     ap.add_argument("-j", type=int, default=min(8, os.cpu_count() or 8))
+    ap.add_argument("--component", choices=sorted(COMPONENTS), default=None)
     a = ap.parse_args(argv)
-    print(build(force=a.force, jobs=a.j, verbose=True))
+    print(build(force=a.force, jobs=a.j, verbose=True, component=a.component))
 
 
 if __name__ == "__main__":

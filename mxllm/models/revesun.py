@@ -149,6 +149,7 @@ class RevesunLayer(nn.Module):
 
 class Revesun(nn.Module):
     serves_float32 = True  # every kernel has an f32 form (mxllm/ops/hybrid.py)
+    native_component = "serve"  # the part of the native library it needs (mxllm/_build.py)
 
     def __init__(self, cfg: RevesunConfig, *, device=None, dtype=torch.bfloat16, seed: int = 0, init: bool = True,
                  lora_r: int = 0, lora_alpha: float = 16.0):

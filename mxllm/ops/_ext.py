@@ -43,6 +43,22 @@ def _load() -> bool:
     return _LOADED
 
 
+def load_component(name: str) -> None:
+    """Have at least component ``name`` (mxllm/_build.py ``COMPONENTS``) loaded: the whole library where it
+    is built, else the component's own, compiled if needed.  For processes that need no other op."""
+    global _LOADED
+    from mxllm import _build
+
+    with _LOCK:
+        if _LOADED:
+            return
+        lib = LIB if os.path.exists(LIB) else _build.COMPONENTS[name][0]
+        if lib != LIB and os.environ.get("MXLLM_NO_AUTOBUILD") != "1":
+            _build.build(jobs=int(os.environ.get("MAX_JOBS", "8")), component=name)  # a no-op when up to date
+        torch.ops.load_library(lib)
+        _LOADED = True
+
+
 def available() -> bool:
     return _load()
 

@@ -100,12 +100,17 @@ def main(argv=None) -> int:
     from ..models import MODEL_CLASSES, model_config
 
     dtype = getattr(torch, a.dtype)
-    if dtype == torch.float32 and not getattr(MODEL_CLASSES[type(model_config(a.model))], "serves_float32", False):
+    cls = MODEL_CLASSES[type(model_config(a.model))]
+    if dtype == torch.float32 and not getattr(cls, "serves_float32", False):
         print("this model's kernels are bfloat16 only", file=sys.stderr)
         return 3
-    from ..ops import native
+    from ..ops import _ext
 
-    native()  # compiles the HIP library if the checkout has none
+    part = getattr(cls, "native_component", None)
+    if part:
+        _ext.load_component(part)  # compiles what the model needs if the checkout has no built library
+    else:
+        _ext.native()
     if not torch.cuda.is_available():
         print("trace_run needs a GPU", file=sys.stderr)
         return 1
