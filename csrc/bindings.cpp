@@ -355,6 +355,7 @@ int64_t cu_masked_stream(int64_t device, std::vector<int64_t> mask) {
   for (size_t i = 0; i < mask.size(); ++i) w[i] = (uint32_t)(mask[i] & 0xffffffffLL);
   hipStream_t s = nullptr;
   hipError_t e = hipExtStreamCreateWithCUMask(&s, (uint32_t)(w.size() * 32), w.data());
+  if (e != hipSuccess) (void)hipGetLastError();  // reported here, not by the next GPU call
   MX_CHECK(e == hipSuccess, "hipExtStreamCreateWithCUMask: ", hipGetErrorString(e));
   return (int64_t)reinterpret_cast<intptr_t>(s);
 }

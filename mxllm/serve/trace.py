@@ -29,7 +29,7 @@ import torch
 from ..models import build_model
 from .engine import Engine
 
-MAX_SLOTS = 1024
+MAX_SLOTS = 256
 
 
 class Replay:
