@@ -191,11 +191,11 @@ __device__ __forceinline__ void conv_taps(const float* w, int n, float (&v)[VEC]
 
 // prompt rows: rows [T] = (position, slot or -1, sequence length, -).  One thread walks RUN consecutive
 // rows of VEC channels with the last taps - 1 rows in registers.
-constexpr int kConvRun = 8;
+constexpr int kConvRun = 4, kConvThreads = 128;
 template <int VEC, typename T, int TAPS>
-__global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, const int4* __restrict__ rows, int T_,
+__global__ void __launch_bounds__(kConvThreads) conv_rope_prefill_kernel(ConvRope a, const int4* __restrict__ rows, int T_,
                                                                 int nvec) {
-  const int f = blockIdx.x * 256 + threadIdx.x;
+  const int f = blockIdx.x * kConvThreads + threadIdx.x;
   if (f >= nvec) return;
   int sec, head, d0, ch, dim;
   conv_where<VEC>(a, f, sec, head, d0, ch, dim);
@@ -223,6 +223,57 @@ __global__ void __launch_bounds__(256) conv_rope_prefill_kernel(ConvRope a, cons
       win[j].load(x + min(max(r0 - (TAPS - 1) + j, 0), T_ - 1) * a.ldx, n);  // rows outside: not used
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) conv_taps<VEC>(a.w + (int64_t)j * C + ch, n, wt[j]);
+    if constexpr (VEC == 8) {
+      // the common run: whole rows inside one sequence, none of them among its last taps, all or none
+      // kept, whole pairs of four: straight-line code, every table read independent of the row before
+      const int4 ra = rows[r0], rb = rows[r1 - 1];
+      const int p0 = ra.x, from = ra.z / a.chunk * a.chunk;
+      const bool keep = ra.y >= 0 && a.kc && p0 >= from;
+      if (r1 - r0 == kConvRun && p0 >= TAPS - 1 && rb.x == p0 + kConvRun - 1 && (a.rd & 7) == 0 && a.rd > 0 &&
+          (ra.y < 0 || !a.kc || (rb.x < ra.z - taps && (keep || rb.x < from)))) {
+        const bool rot = sec < 2 && d0 < a.rd;
+        const int hr = a.rd >> 1, Wp = sec < 2 ? a.Dp : a.Ep;
+        const float* ct = a.cosb + (int64_t)p0 * hr + (rot ? d0 >> 1 : 0);
+        const float* st = a.sinb + (int64_t)p0 * hr + (rot ? d0 >> 1 : 0);
+        const int64_t step = sec == 0 ? a.qt : sec == 1 ? a.kt : a.vt;
+        T* out = reinterpret_cast<T*>(sec == 0 ? a.q : sec == 1 ? a.k : a.v) +
+                 head * (sec == 0 ? a.qh : sec == 1 ? a.kh : a.vh) + r0 * step;
+        const bool last = d0 + VEC >= dim && dim < Wp;
+        auto run = [&](auto keep_c) {
+#pragma unroll
+          for (int k = 0; k < kConvRun; ++k) {
+            float u[VEC], y[VEC], c[4], sn[4];
+            ldv<4>(ct + (int64_t)k * hr, c);
+            ldv<4>(st + (int64_t)k * hr, sn);
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) {
+              win[k + j].get(u);
+#pragma unroll
+              for (int i = 0; i < VEC; ++i) y[i] = j == 0 ? wt[0][i] * u[i] : y[i] + wt[j][i] * u[i];
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const float cc = rot ? c[i] : 1.f, ss = rot ? sn[i] : 0.f, e = y[2 * i], f = y[2 * i + 1];
+              y[2 * i] = e * cc - f * ss;
+              y[2 * i + 1] = f * cc + e * ss;
+            }
+            stv<VEC>(out + k * step + d0, y);
+            if constexpr (decltype(keep_c)::value) {
+              if (sec > 0)
+                stv<VEC>(reinterpret_cast<T*>(sec == 1 ? a.kc : a.vc) +
+                             kv_row(a.bt, a.maxb, a.block, ra.y, a.G, head, p0 - from + k) * Wp + d0,
+                         y);
+            }
+          }
+          if (last)  // the head's padding
+            for (int k = 0; k < kConvRun; ++k)
+              for (int d = dim; d < Wp; ++d) st1(out + k * step + d, 0.f);
+        };
+        if (keep) run(std::true_type{});
+        else run(std::false_type{});
+        return;
+      }
+    }
 #pragma unroll
     for (int k = 0; k < kConvRun; ++k) {
       const int r = r0 + k;
@@ -448,7 +499,7 @@ extern "C" int mx_conv_rope_prefill(const ConvRope* pa, int f32, const int32_t* 
   const ConvRope& a = *pa;
   if (conv_check(a)) return -1;
 #define CP(VV, TT, TP)                                                                             \
-  conv_rope_prefill_kernel<VV, TT, TP><<<dim3((conv_nvec<VV>(a) + 255) / 256, (T + kConvRun - 1) / kConvRun), 256, \
+  conv_rope_prefill_kernel<VV, TT, TP><<<dim3((conv_nvec<VV>(a) + kConvThreads - 1) / kConvThreads, (T + kConvRun - 1) / kConvRun), kConvThreads, \
                                          0, stream>>>(a, (const int4*)rows, T, conv_nvec<VV>(a))
 #define CPT(VV, TT)                                                                                \
   if (a.taps == 4) CP(VV, TT, 4); else if (a.taps == 3) CP(VV, TT, 3); else if (a.taps == 2) CP(VV, TT, 2); \
