@@ -1,9 +1,9 @@
 // Torch op registrations for the mxllm HIP kernels (namespace torch.ops.mxllm).
 //
 // Kernels live in csrc/kernels/*.hip and expose plain C launchers
-// (`mx_*`, taking raw pointers + hipStream_t); this file is the only one that
-// includes torch headers, so kernel files compile in seconds and stay free of
-// ATen.  Every op runs on the current HIP stream of the input's device.
+// (`mx_*`, taking raw pointers + hipStream_t); only the bindings*.cpp files
+// include torch headers, so kernel files compile in seconds and stay free of
+// ATen (serving ops: bindings_serve.cpp, bindings_hybrid.cpp).  Every op runs on the current HIP stream of the input's device.
 #include "bindings_util.h"
 
 namespace {

@@ -243,7 +243,8 @@ def build_default(model: str = "tiny", device: str | None = None, max_batch: int
 def main(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--model", default=os.environ.get("MXLLM_MODEL", "tiny"),
-                    help="preset name, or a Hugging Face Llama directory (config.json + safetensors + tokenizer.json)")
+                    help="preset name, or a model directory (config.json + safetensors [+ tokenizer.json]): Hugging Face "
+                         "Llama, or a design config.json names")
     ap.add_argument("--host", default="127.0.0.1")
     ap.add_argument("--port", type=int, default=8000)
     ap.add_argument("--max-batch", type=int, default=8)
